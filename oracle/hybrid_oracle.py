@@ -1,8 +1,8 @@
 """Plain, slow restatement of the mechanisms of config-described hybrid decoders, on CPU tensors.
 
 TEST INFRASTRUCTURE, NOT PRODUCT.  One function per mechanism, written from the equations with explicit loops over
-tokens and keys; float64 by default.  `gafulix_logits` composes them for a checkpoint given as (config dictionary,
-{tensor name: tensor}).  Nothing here is imported by the product and nothing of the product is imported here."""
+tokens and keys; float64 by default.  `gafulix_logits` and `roletar_logits` compose them for a checkpoint given as
+(config dictionary, {tensor name: tensor}).  Nothing here is imported by the product and nothing of the product is imported here."""
 from __future__ import annotations
 
 import math
@@ -51,23 +51,26 @@ def rotate_interleaved(x, position, freqs, magnitude, dims):
 
 
 # ---- attention --------------------------------------------------------------------------------------------------
-def visible(i, j, chunk=None):
+def visible(i, j, chunk=None, window=None):
     """Whether the token at position i sees the key at position j."""
-    return j <= i and (not chunk or i // chunk == j // chunk)
+    return j <= i and (not chunk or i // chunk == j // chunk) and (not window or i - j < window)
 
 
-def attend(q, k, v, scale, chunk=None):
-    """q [T, H, dim], k [T, G, dim], v [T, G, vdim] of one sequence from position 0; returns [T, H, vdim]."""
+def attend(q, k, v, scale, chunk=None, window=None, sink=None):
+    """q [T, H, dim], k [T, G, dim], v [T, G, vdim] of one sequence from position 0; returns [T, H, vdim].
+    sink [H]: a further, unscaled score per head whose share of the softmax goes nowhere."""
     T, H, _ = q.shape
     G = k.shape[1]
     out = torch.zeros(T, H, v.shape[2], dtype=q.dtype)
     for i in range(T):
-        js = [j for j in range(T) if visible(i, j, chunk)]
+        js = [j for j in range(T) if visible(i, j, chunk, window)]
         for h in range(H):
             g = h // (H // G)
             s = (k[js, g] @ q[i, h]) * scale
-            p = torch.exp(s - s.max())
-            out[i, h] = (p / p.sum()) @ v[js, g]
+            top = s.max() if sink is None else torch.maximum(s.max(), sink[h])
+            p = torch.exp(s - top)
+            total = p.sum() if sink is None else p.sum() + torch.exp(sink[h] - top)
+            out[i, h] = (p / total) @ v[js, g]
     return out
 
 
@@ -84,6 +87,69 @@ def attention_mixer(h, w, cfg, eps):
         k = torch.stack([rotate_interleaved(k[t], t, freqs, mag, rot["dims"]) for t in range(T)])
     chunk = (cfg.get("mask") or {}).get("size")
     return attend(q, k, v, cfg["scale"], chunk).reshape(T, H * vdim) @ w["o"].T
+
+
+def sink_attention_mixer(h, w, cfg, eps):
+    """Grouped heads without rotation, a sliding window, a sink per head."""
+    T = h.shape[0]
+    H, G, dim, vdim = cfg["heads"], cfg["kv_heads"], cfg["dim"], cfg["vdim"]
+    q, k, v = (h @ w["q"].T).view(T, H, dim), (h @ w["k"].T).view(T, G, dim), (h @ w["v"].T).view(T, G, vdim)
+    window = (cfg.get("mask") or {}).get("size")
+    return attend(q, k, v, cfg["scale"], window=window, sink=w["sink"]).reshape(T, H * vdim) @ w["o"].T
+
+
+def latent_attention_mixer(h, w, cfg, eps):
+    """Keys and values of all heads from one normalised latent per token, plus one rotated key part that the heads share."""
+    T = h.shape[0]
+    H, dim, rd, vdim, rank = cfg["heads"], cfg["dim"], cfg["rot_dim"], cfg["vdim"], cfg["kv_rank"]
+    freqs, mag = rotary_frequencies(rd, cfg["rot"]["base"])
+    q = (h @ w["q"].T).view(T, H, dim + rd)
+    down = h @ w["dkv"].T
+    latent = rms(down[:, :rank], w["dkv.norm"], eps)
+    k_nope, v = (latent @ w["uk"].T).view(T, H, dim), (latent @ w["uv"].T).view(T, H, vdim)
+    keys, queries = [], []
+    for t in range(T):
+        k_rot = rotate_interleaved(down[t:t + 1, rank:], t, freqs, mag, rd)
+        keys.append(torch.cat([k_nope[t], k_rot.expand(H, rd)], dim=1))
+        queries.append(torch.cat([q[t, :, :dim], rotate_interleaved(q[t, :, dim:], t, freqs, mag, rd)], dim=1))
+    return attend(torch.stack(queries), torch.stack(keys), v, cfg["scale"]).reshape(T, H * vdim) @ w["o"].T
+
+
+# ---- selective scan (Gu and Dao, "Mamba: Linear-Time Sequence Modeling with Selective State Spaces") -------------------
+def short_conv(x, weight, bias, before=None):
+    """x [T, C], weight [C, taps] (last column: the current token), `before` [taps - 1, C]: the inputs ahead of x (zeros)."""
+    T, C = x.shape
+    taps = weight.shape[1]
+    padded = torch.cat([torch.zeros(taps - 1, C, dtype=x.dtype) if before is None else before, x])
+    out = bias.expand(T, C).clone()
+    for k in range(taps):
+        out = out + weight[:, k] * padded[k:k + T]
+    return out
+
+
+def softplus(z):
+    return torch.clamp(z, min=0.0) + torch.log1p(torch.exp(-z.abs()))
+
+
+def selective_scan(x, dt, A, B, C, D, state=None):
+    """x, dt [T, channels], A [channels, N] (negative), B, C [T, N], D [channels]; state [channels, N] (zero if not given).
+    Returns (y [T, channels], the state after the last token)."""
+    S = torch.zeros_like(A) if state is None else state.clone()
+    out = torch.zeros_like(x)
+    for t in range(x.shape[0]):
+        S = torch.exp(dt[t, :, None] * A) * S + (dt[t] * x[t])[:, None] * B[t]
+        out[t] = S @ C[t] + D * x[t]
+    return out, S
+
+
+def mamba1_mixer(h, w, cfg, eps):
+    inner, rank, n = cfg["inner"], cfg["dt_rank"], cfg["state"]
+    x, z = (h @ w["in"].T).split([inner, inner], dim=1)
+    x = silu(short_conv(x, w["conv"], w["conv.b"]))
+    low, B, C = (x @ w["x"].T).split([rank, n, n], dim=1)
+    dt = softplus(low @ w["dt"].T + w["dt.b"])
+    y, _ = selective_scan(x, dt, -torch.exp(w["A_log"]), B, C, w["D"])
+    return (y * silu(z)) @ w["o"].T
 
 
 # ---- gated linear attention -------------------------------------------------------------------------------------
@@ -136,6 +202,26 @@ def moe(h, w, cfg):
     return out
 
 
+def relu2_mlp(h, w):
+    return torch.clamp(h @ w["up"].T, min=0.0) ** 2 @ w["down"].T
+
+
+# ---- hyper-connections -------------------------------------------------------------------------------------------
+def hyper_read(xs, w_in):
+    """The input of a sublayer from the streams xs [S, T, width]."""
+    return sum(w_in[s] * xs[s] for s in range(len(xs)))
+
+
+def hyper_write(xs, mix, w_out, y):
+    """Every stream anew from all the old ones (mix[from, to]) and the sublayer's output."""
+    n = len(xs)
+    return torch.stack([sum(mix[s, t] * xs[s] for s in range(n)) + w_out[t] * y for t in range(n)])
+
+
+def softcap(logits, cap):
+    return cap * torch.tanh(logits / cap)
+
+
 # ---- the model --------------------------------------------------------------------------------------------------
 def layer_schedule(config):
     """[(layer index, whether the embedding output is added in front of it)] in execution order."""
@@ -174,3 +260,26 @@ def gafulix_logits(config, weights, tokens, dtype=torch.float64, trace=None):
         if trace is not None:
             trace.append(x.clone())
     return rms(x, w("final.norm"), eps) @ w("head").T
+
+
+def roletar_logits(config, weights, tokens, dtype=torch.float64, trace=None):
+    """As gafulix_logits.  `trace` receives the sum of the streams."""
+    eps = config["norm"]["eps"]
+    w = lambda name: weights[name].to(dtype)
+    emb = w("embed")[torch.tensor(tokens)]
+    xs = torch.stack([emb] * config["streams"])
+    for i, _ in layer_schedule(config):
+        layer = config["layers"][i]
+        mix = _sub(weights, f"l{i}.mix.", dtype)
+        mixer = {"attention": sink_attention_mixer, "latent_attention": latent_attention_mixer,
+                 "mamba1": mamba1_mixer}[layer["type"]]
+        subs = [("1", lambda h: mixer(h, mix, layer["mixer"], eps))]
+        if layer.get("mlp"):
+            subs.append(("2", lambda h: relu2_mlp(h, _sub(weights, f"l{i}.mlp.", dtype))))
+        for n, f in subs:
+            hc = _sub(weights, f"l{i}.hc{n}.", dtype)
+            y = f(rms(hyper_read(xs, hc["in"]), w(f"l{i}.norm{n}"), eps))
+            xs = hyper_write(xs, hc["mix"], hc["out"], y)
+        if trace is not None:
+            trace.append(xs.sum(dim=0))
+    return softcap(rms(xs.sum(dim=0), w("final.norm"), eps) @ w("head").T, config["logit_softcap"])
