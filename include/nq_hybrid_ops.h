@@ -1,7 +1,8 @@
 /* C ABI of libnq_hybrid.so: the kernels of decoders that a configuration describes layer by layer -- sandwich norms on
- * an fp32 residual stream, attention with whole-projection q/k norm, interleaved rotary and a chunked mask over the
- * paged KV cache, gated linear attention with an fp32 recurrent state, mixtures of experts with an input-side weight,
- * dense skinny products, and the bookkeeping of a decode step.
+ * an fp32 residual stream, attention with whole-projection q/k norm, interleaved rotary, a chunked or sliding-window mask
+ * and sinks over the paged KV cache, gated linear attention with an fp32 recurrent state, mixtures of experts with an input-side weight,
+ * latent attention, selective scans with a short convolution, residuals of several streams (hyper-connections), dense
+ * skinny products, and the bookkeeping of a decode step.
  *
  * Conventions: device pointers, dense row-major tensors unless a row stride is given, `dtype` is NQH_BF16 or NQH_F32
  * for every activation and weight of a call, `stream` is a hipStream_t as void*.  The return value is 0 or an NQH_ERR
@@ -20,6 +21,9 @@ extern "C" {
 enum nqh_dtype { NQH_BF16 = 1, NQH_F32 = 2 };
 enum nqh_status { NQH_OK = 0, NQH_ERR_ARG = 1, NQH_ERR_UNSUPPORTED = 2, NQH_ERR_WORKSPACE = 3, NQH_ERR_HIP = 4 };
 
+/* What follows a matrix product: nothing, the square of max(v, 0), or param * tanh(v / param). */
+enum nqh_activation { NQH_ACT_NONE = 0, NQH_ACT_RELU2 = 1, NQH_ACT_SOFTCAP = 2 };
+
 const char* nqh_last_error(void);
 
 /* The step between two sublayers, on the fp32 residual stream x [rows, width]:
@@ -31,6 +35,20 @@ const char* nqh_last_error(void);
 int nqh_residual_norm(float* x, int init, const void* y, int64_t y_parts, const void* post_weight, const int64_t* ids,
                       const void* table, int64_t table_rows, const void* next_weight, void* h, int64_t rows,
                       int64_t width, float eps, int dtype, void* stream);
+
+/* The step between two sublayers with hyper-connections, on the fp32 residual x [rows, streams, width]:
+ *   x[., s]  = table[ids[r]] for every stream s                              (ids given: the start; y must be NULL)
+ *   x[., t]  = sum_s mix[s, t] x[., s] + w_out[t] y, all at once             (y [rows, width] may be NULL)
+ *   h        = RMSNorm(sum_s w_in[s] x[., s]) * norm_weight                  (h may be NULL; w_in NULL: ones)
+ * mix [streams, streams], w_out and w_in [streams] have the call's dtype.  width <= 8192, streams <=
+ * nqh_hyper_max_streams. */
+int64_t nqh_hyper_max_streams(void);
+int nqh_hyper_norm(float* x, const int64_t* ids, const void* table, int64_t table_rows, const void* y, const void* mix,
+                   const void* w_out, const void* w_in, const void* norm_weight, void* h, int64_t rows, int64_t streams,
+                   int64_t width, float eps, int dtype, void* stream);
+
+/* x [count] = activation(x), in place; act is an nqh_activation. */
+int nqh_activate(void* x, int64_t count, int act, float param, int dtype, void* stream);
 
 /* nqh_residual_norm with the router and the plan of the layer behind it in the same launch, for few rows (see
  * nqh_residual_norm_route_supported): h as above (required), expert / weight as nqh_router_topk on h, order / tiles as
@@ -57,25 +75,101 @@ int nqh_qk_norm_rope_store(const void* qkv, const void* q_weight, const void* k_
 /* Attention of the query tokens of a prompt pass over their sequences' cached keys (their own included).  The pass is a
  * list of segments, int32 [.][3] = first row in q, rows, position of the first row in its sequence; segment s has the block
  * table block_tables[s] (int32 [.][max_blocks]).  A query at position i sees key j when j <= i and, if chunk > 0,
- * i / chunk == j / chunk.  Work is dealt by the tile list, int32 [num_tiles][2] = segment, first row inside it; a tile
+ * i / chunk == j / chunk and, if window > 0, i - j < window.  sink [heads] (may be NULL): a term exp(sink[h]) in the
+ * denominator of the softmax.  Work is dealt by the tile list, int32 [num_tiles][2] = segment, first row inside it; a tile
  * covers nqh_attention_tile_rows rows.  q [rows, heads, k_row], out [rows, heads * vdim].
  * The positions of every segment must lie inside its block table. */
 int64_t nqh_attention_tile_rows(void);
 int nqh_attention_prefill(const void* q, const void* k_cache, const void* v_cache, const int32_t* block_tables,
-                          const int32_t* segments, const int32_t* tiles, void* out, int64_t rows, int64_t num_tiles,
-                          int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim, int64_t k_row, int64_t v_row,
-                          int64_t block_size, int64_t max_blocks, int64_t num_blocks, int64_t chunk, float scale, int dtype,
-                          void* stream);
+                          const int32_t* segments, const int32_t* tiles, const void* sink, void* out, int64_t rows,
+                          int64_t num_tiles, int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim, int64_t k_row,
+                          int64_t v_row, int64_t block_size, int64_t max_blocks, int64_t num_blocks, int64_t chunk,
+                          int64_t window, float scale, int dtype, void* stream);
 
 /* The same for one new token of each of `batch` sequences: context_lens[b] tokens are cached, the query is the last of
  * them.  block_table int32 [batch, max_blocks].  Workspace: nqh_attention_decode_workspace_bytes, uninitialised. */
 size_t nqh_attention_decode_workspace_bytes(int64_t batch, int64_t heads, int64_t kv_heads, int64_t v_row,
-                                            int64_t max_context, int64_t chunk, int dtype);
+                                            int64_t max_context, int64_t chunk, int64_t window, int dtype);
 int nqh_attention_decode(const void* q, const void* k_cache, const void* v_cache, const int32_t* block_table,
-                         const int32_t* context_lens, void* out, int64_t batch, int64_t heads, int64_t kv_heads,
-                         int64_t dim, int64_t vdim, int64_t k_row, int64_t v_row, int64_t block_size, int64_t max_blocks,
-                         int64_t num_blocks, int64_t chunk, float scale, int dtype, void* workspace,
+                         const int32_t* context_lens, const void* sink, void* out, int64_t batch, int64_t heads,
+                         int64_t kv_heads, int64_t dim, int64_t vdim, int64_t k_row, int64_t v_row, int64_t block_size,
+                         int64_t max_blocks, int64_t num_blocks, int64_t chunk, int64_t window, float scale, int dtype, void* workspace,
                          size_t workspace_bytes, void* stream);
+
+/* Latent attention.  A token's cache row [block][token][row] holds its normalised latent (rank elements) and, at rot_at, the
+ * rotated key part (rot_dim) that all heads share; the rest of the row stays zero.
+ * nqh_latent_store: proj [rows, heads * (dim + rot_dim) + rank + rot_dim] = the heads' queries [dim | rot_dim], latent,
+ * rotated key part.  The latent is RMS-normalised with norm_weight [rank], the rotated parts of queries and key turn pairs
+ * (2i, 2i + 1) by cos_sin [max_positions, rot_dim] = cos | sin at positions[row]; latent and key part go to the cache row
+ * slots[row] (outside [0, num_slots): not written).  q_out [rows, heads, q_row] receives the rotated part at rot_q and, with
+ * copy_plain, the unrotated part at 0; what lies beyond dim (without copy_plain: beyond rank, which nqh_head_linear fills) is
+ * zeroed. */
+int nqh_latent_store(const void* proj, const void* norm_weight, const float* cos_sin, const int64_t* positions,
+                     const int64_t* slots, void* q_out, void* cache, int64_t rows, int64_t heads, int64_t dim,
+                     int64_t rot_dim, int64_t rank, int64_t q_row, int64_t rot_q, int copy_plain, int64_t row,
+                     int64_t rot_at, int64_t max_positions, int64_t num_slots, float eps, int dtype, void* stream);
+
+/* The contexts of all segments (see nqh_attention_prefill; at most `longest` tokens each) from the cache to consecutive
+ * rows without padding: out [., rank + rot_dim], segment s from row first[s] on.  2-byte elements; sizes multiples of 8. */
+int nqh_latent_gather(const void* cache, const int32_t* tables, const int32_t* segments, const int32_t* first, void* out,
+                      int64_t num_segments, int64_t longest, int64_t rank, int64_t rot_dim, int64_t row, int64_t rot_at,
+                      int64_t block_size, int64_t max_blocks, int64_t num_blocks, void* stream);
+
+/* y[r, h, :] = weight[h] x[r, h, :] with weight [heads, out, in]; x_row, x_head, y_row, y_head: elements between rows and
+ * between heads. */
+int nqh_head_linear(const void* x, const void* weight, void* y, int64_t rows, int64_t heads, int64_t out_features,
+                    int64_t in_features, int64_t x_row, int64_t x_head, int64_t y_row, int64_t y_head, int dtype,
+                    void* stream);
+
+/* Prompt attention over keys and values expanded per head, bf16: token j of segment s is row first[s] + j of kv [.,
+ * kv_stride] = heads x dim unrotated keys, then heads x vdim values, and of rot [., rot_stride], the shared rotated part.
+ * q [rows, heads, q_row] with q_row = nqh_latent_attention_prefill_query_row (0: these sizes are not supported); segments and
+ * tiles as in nqh_attention_prefill; causal. */
+int64_t nqh_latent_attention_prefill_query_row(int64_t dim, int64_t rot_dim, int64_t vdim, int dtype);
+int nqh_latent_attention_prefill(const void* q, const void* kv, int64_t kv_stride, const void* rot, int64_t rot_stride,
+                                 const int32_t* first, const int32_t* segments, const int32_t* tiles, void* out, int64_t rows,
+                                 int64_t num_tiles, int64_t heads, int64_t dim, int64_t rot_dim, int64_t vdim, float scale,
+                                 void* stream);
+
+/* Decode attention over the latents themselves: q [batch, heads, row] = queries multiplied into the latent space, with the
+ * rotated part at rot_at; out [batch, heads, rank] is still in the latent space.  In bf16 rot_at 64, 128, 256 or 512 with row
+ * - rot_at 32 or 64 runs on the matrix cores, anything else (row <= 1024, rank <= 512) on the vector ALU. */
+size_t nqh_latent_attention_decode_workspace_bytes(int64_t batch, int64_t heads, int64_t rank, int64_t rot_at, int64_t row,
+                                                   int64_t max_context, int dtype);
+int nqh_latent_attention_decode(const void* q, const void* cache, const int32_t* block_table, const int32_t* context_lens,
+                                void* out, int64_t batch, int64_t heads, int64_t rank, int64_t rot_at, int64_t row,
+                                int64_t block_size, int64_t max_blocks, int64_t num_blocks, float scale, int dtype,
+                                void* workspace, size_t workspace_bytes, void* stream);
+
+/* Selective scan.  Per channel c and state n: S[n, c] = exp(dt[c] A[c, n]) S[n, c] + dt[c] x[c] B[n], y[c] =
+ * (sum_n S[n, c] C[n] + D[c] x[c]) silu(z[c]), A = -exp(a_log [channels, states]).  x is the output of a causal convolution
+ * per channel (weight [channels, taps], last column: the current token) with bias and silu.  state fp32 [slots, states,
+ * channels], tail fp32 [slots, taps - 1, channels]: the convolution's last inputs, oldest first; neither is ever cleared,
+ * before position 0 both count as zero.  bc rows hold B | C.  *_stride: elements between rows.
+ * Pieces of a pass as in nqh_gla_prefill (nqh_scan_piece_rows: a good size, the least allowed is what it gives for one row);
+ * longest: rows of the longest piece.  At most 256 states and 16 taps. */
+int nqh_conv_silu(const void* x, int64_t x_stride, const void* weight, const void* bias, const float* tail,
+                  const int32_t* pieces, int64_t num_pieces, int64_t longest, void* out, int64_t channels, int64_t taps,
+                  int dtype, void* stream);
+int nqh_conv_step(const void* x, int64_t x_stride, const void* weight, const void* bias, float* tail,
+                  const int32_t* state_slots, const int64_t* positions, const uint8_t* active, void* out, int64_t batch,
+                  int64_t num_slots, int64_t channels, int64_t taps, int dtype, void* stream);
+/* dt [rows, channels] = log(1 + exp(weight [channels, rank] low + bias)), fp32. */
+int nqh_scan_dt(const void* low, int64_t low_stride, const void* weight, const void* bias, float* dt, int64_t rows,
+                int64_t channels, int64_t rank, int dtype, void* stream);
+/* The pass's tokens through the recurrence; conv_in: the convolution's inputs, from which the tail is taken.  out [rows,
+ * channels].  chained: some sequence has several pieces (the workspace is needed then, uninitialised). */
+int64_t nqh_scan_piece_rows(int64_t rows, int64_t channels, int64_t states);
+size_t nqh_scan_workspace_bytes(int64_t num_pieces, int64_t channels, int64_t states);
+int nqh_scan_prefill(const void* x, const float* dt, const void* bc, int64_t bc_stride, const void* z, int64_t z_stride,
+                     const void* a_log, const void* d_skip, const void* conv_in, int64_t conv_stride, float* state, float* tail,
+                     const int32_t* pieces, int64_t num_pieces, int chained, void* out, int64_t channels, int64_t states,
+                     int64_t taps, int dtype, void* workspace, size_t workspace_bytes, void* stream);
+/* One token of each sequence; idle rows and slots as in nqh_gla_decode. */
+int nqh_scan_step(const void* x, const float* dt, const void* bc, int64_t bc_stride, const void* z, int64_t z_stride,
+                  const void* a_log, const void* d_skip, float* state, const int32_t* state_slots, const int64_t* positions,
+                  const uint8_t* active, void* out, int64_t batch, int64_t num_slots, int64_t channels, int64_t states,
+                  int dtype, void* stream);
 
 /* decay[r, c] = sigmoid(low[r, :] . up[c, :] + bias[c])^(1 / tau), fp32; low [rows, rank] with row stride low_stride,
  * up [channels, rank]. */
@@ -135,9 +229,10 @@ int nqh_moe_down(const void* act, const void* down, const int32_t* order, const 
                  int64_t experts, int64_t width, int64_t ff, int64_t tile_rows, int64_t max_tiles, int dtype,
                  void* stream);
 
-/* y [rows, out] = x [rows, in] weight[out, in]^T (+ bias) for few rows (<= 64), bf16 operands; y in fp32 if out_f32. */
+/* y [rows, out] = act(x [rows, in] weight[out, in]^T (+ bias)) for few rows (<= 64), bf16 operands; y in fp32 if out_f32;
+ * act and param as in nqh_activate. */
 int nqh_skinny_linear(const void* x, const void* weight, const void* bias, void* y, int64_t rows, int64_t out_features,
-                      int64_t in_features, int out_f32, void* stream);
+                      int64_t in_features, int out_f32, int act, float param, void* stream);
 
 /* Decode-step bookkeeping, as nq_argmax_rows / nq_decode_prepare / nq_decode_advance (nq_engine_ops.h) do it; the
  * logits are fp32. */

@@ -86,9 +86,27 @@ HYBRID_SYMBOLS = {
     "nqh_residual_norm_route": (_int, [_vp, _int, _vp, _i64, _vp, _vp, _vp, _i64] + [_vp] * 8 + [_i64] * 6 + [_f32, _int, _vp]),
     "nqh_qk_norm_rope_store": (_int, [_vp] * 9 + [_i64] * 11 + [_f32, _int, _vp]),
     "nqh_attention_tile_rows": (_i64, []),
-    "nqh_attention_prefill": (_int, [_vp] * 7 + [_i64] * 12 + [_f32, _int, _vp]),
-    "nqh_attention_decode_workspace_bytes": (_sz, [_i64] * 6 + [_int]),
-    "nqh_attention_decode": (_int, [_vp] * 6 + [_i64] * 11 + [_f32, _int, _vp, _sz, _vp]),
+    "nqh_attention_prefill": (_int, [_vp] * 8 + [_i64] * 13 + [_f32, _int, _vp]),
+    "nqh_attention_decode_workspace_bytes": (_sz, [_i64] * 7 + [_int]),
+    "nqh_attention_decode": (_int, [_vp] * 7 + [_i64] * 12 + [_f32, _int, _vp, _sz, _vp]),
+    "nqh_hyper_max_streams": (_i64, []),
+    "nqh_hyper_norm": (_int, [_vp] * 3 + [_i64] + [_vp] * 6 + [_i64] * 3 + [_f32, _int, _vp]),
+    "nqh_activate": (_int, [_vp, _i64, _int, _f32, _int, _vp]),
+    "nqh_latent_store": (_int, [_vp] * 7 + [_i64] * 7 + [_int] + [_i64] * 4 + [_f32, _int, _vp]),
+    "nqh_latent_gather": (_int, [_vp] * 5 + [_i64] * 9 + [_vp]),
+    "nqh_head_linear": (_int, [_vp] * 3 + [_i64] * 8 + [_int, _vp]),
+    "nqh_latent_attention_prefill_query_row": (_i64, [_i64] * 3 + [_int]),
+    "nqh_latent_attention_prefill": (_int, [_vp, _vp, _i64, _vp, _i64] + [_vp] * 4 + [_i64] * 6 + [_f32, _vp]),
+    "nqh_latent_attention_decode_workspace_bytes": (_sz, [_i64] * 6 + [_int]),
+    "nqh_latent_attention_decode": (_int, [_vp] * 5 + [_i64] * 8 + [_f32, _int, _vp, _sz, _vp]),
+    "nqh_conv_silu": (_int, [_vp, _i64] + [_vp] * 4 + [_i64] * 2 + [_vp] + [_i64] * 2 + [_int, _vp]),
+    "nqh_conv_step": (_int, [_vp, _i64] + [_vp] * 7 + [_i64] * 4 + [_int, _vp]),
+    "nqh_scan_dt": (_int, [_vp, _i64] + [_vp] * 3 + [_i64] * 3 + [_int, _vp]),
+    "nqh_scan_piece_rows": (_i64, [_i64] * 3),
+    "nqh_scan_workspace_bytes": (_sz, [_i64] * 3),
+    "nqh_scan_prefill": (_int, [_vp, _vp, _vp, _i64, _vp, _i64, _vp, _vp, _vp, _i64, _vp, _vp, _vp, _i64, _int, _vp] + [_i64] * 3
+                         + [_int, _vp, _sz, _vp]),
+    "nqh_scan_step": (_int, [_vp, _vp, _vp, _i64, _vp, _i64] + [_vp] * 7 + [_i64] * 4 + [_int, _vp]),
     "nqh_gla_decay": (_int, [_vp, _i64, _vp, _vp, _vp, _i64, _i64, _i64, _f32, _int, _vp]),
     "nqh_gla_piece_rows": (_i64, [_i64] * 4),
     "nqh_gla_prefill_workspace_bytes": (_sz, [_i64] * 4),
@@ -101,7 +119,7 @@ HYBRID_SYMBOLS = {
     "nqh_moe_tile_rows": (_i64, [_i64] * 4 + [_int]),
     "nqh_moe_gate_up": (_int, [_vp] * 6 + [_i64] * 7 + [_int, _vp]),
     "nqh_moe_down": (_int, [_vp] * 5 + [_i64] * 6 + [_int, _vp]),
-    "nqh_skinny_linear": (_int, [_vp] * 4 + [_i64] * 3 + [_int, _vp]),
+    "nqh_skinny_linear": (_int, [_vp] * 4 + [_i64] * 3 + [_int, _int, _f32, _vp]),
     "nqh_argmax_rows": (_int, [_vp, _vp, _i64, _i64, _vp]),
     "nqh_decode_prepare": (_int, [_vp] * 5 + [_i64] * 3 + [_vp]),
     "nqh_decode_advance": (_int, [_vp] * 6 + [_i64] * 2 + [_vp]),

@@ -1,4 +1,4 @@
-// Dense linear for few rows: y = x W^T (+ bias), bf16 operands, fp32 accumulation.
+// Dense linear for few rows: y = act(x W^T (+ bias)), bf16 operands, fp32 accumulation.
 //   up to 16 rows    skinny_linear_kernel: both operands straight from memory, the waves split the contraction
 //   17 to 64 rows    wide_linear_kernel: the activations, by now as many bytes per workgroup as its weights, go through LDS
 #include "skinny.hpp"
@@ -9,7 +9,7 @@ namespace {
 template <bool F32OUT>
 __global__ __launch_bounds__(1024) void skinny_linear_kernel(const uint16_t* __restrict__ x, const uint16_t* __restrict__ w,
                                                              const uint16_t* __restrict__ bias, void* __restrict__ y,
-                                                             int rows, int n_out, int n_in) {
+                                                             int rows, int n_out, int n_in, int act, float param) {
     extern __shared__ __attribute__((aligned(16))) float s_sum[];
     const int lane = threadIdx.x & 63, lo = lane & 15, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int waves = blockDim.x >> 6, n0 = blockIdx.x * 16;
@@ -20,7 +20,7 @@ __global__ __launch_bounds__(1024) void skinny_linear_kernel(const uint16_t* __r
     skinny_reduce<1, 1>(acc, s_sum, wave, waves);
     const int t = threadIdx.x >> 4, n = n0 + (threadIdx.x & 15);
     if (threadIdx.x < 256 && t < rows && n < n_out) {
-        const float v = s_sum[threadIdx.x] + (bias ? Bf::to_f32(bias[n]) : 0.f);
+        const float v = activation_f32(s_sum[threadIdx.x] + (bias ? Bf::to_f32(bias[n]) : 0.f), act, param);
         if constexpr (F32OUT) reinterpret_cast<float*>(y)[(int64_t)t * n_out + n] = v;
         else reinterpret_cast<uint16_t*>(y)[(int64_t)t * n_out + n] = Bf::from_f32(v);
     }
@@ -37,7 +37,7 @@ __device__ const u32x4 g_zero_piece = {0u, 0u, 0u, 0u};   // what lies past the 
 template <int MT, int NT, bool F32OUT>
 __global__ __launch_bounds__(512) void wide_linear_kernel(const uint16_t* __restrict__ x, const uint16_t* __restrict__ w,
                                                           const uint16_t* __restrict__ bias, void* __restrict__ y, int rows,
-                                                          int n_out, int n_in) {
+                                                          int n_out, int n_in, int act, float param) {
     constexpr int KS = 8 / NT, kPart = 16 * MT * 256, kBuf = KS * kPart, kLoads = kBuf / 1024 / 8;
     extern __shared__ __attribute__((aligned(1024))) unsigned char s_x[];   // [buffer][part][row][256 bytes]
     const int lane = threadIdx.x & 63, lo = lane & 15, hi = lane >> 4;
@@ -93,6 +93,7 @@ __global__ __launch_bounds__(512) void wide_linear_kernel(const uint16_t* __rest
         float v = bias ? Bf::to_f32(bias[n]) : 0.f;
 #pragma unroll
         for (int p = 0; p < KS; ++p) v += sums[p * NT * MT * 256 + i];
+        v = activation_f32(v, act, param);
         if constexpr (F32OUT) reinterpret_cast<float*>(y)[(int64_t)t * n_out + n] = v;
         else reinterpret_cast<uint16_t*>(y)[(int64_t)t * n_out + n] = Bf::from_f32(v);
     }
@@ -100,7 +101,7 @@ __global__ __launch_bounds__(512) void wide_linear_kernel(const uint16_t* __rest
 
 template <int MT, int NT>
 int launch_wide(const char* fn, const void* x, const void* w, const void* bias, void* y, int64_t rows, int64_t n_out,
-                int64_t n_in, int out_f32, void* stream) {
+                int64_t n_in, int out_f32, int act, float param, void* stream) {
     constexpr int lds = 2 * (8 / NT) * 16 * MT * 256;
     const auto kernel = out_f32 ? wide_linear_kernel<MT, NT, true> : wide_linear_kernel<MT, NT, false>;
     if (lds > 65536) {
@@ -108,7 +109,7 @@ int launch_wide(const char* fn, const void* x, const void* w, const void* bias, 
         if (e != hipSuccess) return fail(NQH_ERR_HIP, fn, "%s", hipGetErrorString(e));
     }
     kernel<<<dim3((unsigned)cdiv(n_out, 16 * NT)), dim3(512), lds, (hipStream_t)stream>>>(
-        (const uint16_t*)x, (const uint16_t*)w, (const uint16_t*)bias, y, (int)rows, (int)n_out, (int)n_in);
+        (const uint16_t*)x, (const uint16_t*)w, (const uint16_t*)bias, y, (int)rows, (int)n_out, (int)n_in, act, param);
     return launched(fn);
 }
 
@@ -118,21 +119,24 @@ int launch_wide(const char* fn, const void* x, const void* w, const void* bias, 
 using namespace nqh;
 
 extern "C" int nqh_skinny_linear(const void* x, const void* weight, const void* bias, void* y, int64_t rows,
-                                 int64_t out_features, int64_t in_features, int out_f32, void* stream) {
+                                 int64_t out_features, int64_t in_features, int out_f32, int act, float param,
+                                 void* stream) {
     const char* fn = "nqh_skinny_linear";
     if (!x || !weight || !y || !aligned(x, 16) || !aligned(weight, 16))
         return fail(NQH_ERR_ARG, fn, "null or misaligned pointer");
     if (rows <= 0 || rows > 64 || out_features <= 0 || in_features <= 0 || in_features % 8 != 0 ||
         out_features > kMaxI32 - 16 || in_features > (1 << 30))
         return fail(NQH_ERR_ARG, fn, "1 to 64 rows and an in_features that is a multiple of 8");
+    if (act < NQH_ACT_NONE || act > NQH_ACT_SOFTCAP || (act == NQH_ACT_SOFTCAP && !(param > 0.f)))
+        return fail(NQH_ERR_ARG, fn, "unknown activation, or a cap that is not positive");
     (void)hipGetLastError();
     if (rows > 16) {
         const bool narrow = out_features <= 8192;      // fewer features per workgroup: more workgroups
         if (rows <= 32)
-            return narrow ? launch_wide<2, 2>(fn, x, weight, bias, y, rows, out_features, in_features, out_f32, stream)
-                          : launch_wide<2, 4>(fn, x, weight, bias, y, rows, out_features, in_features, out_f32, stream);
-        return narrow ? launch_wide<4, 2>(fn, x, weight, bias, y, rows, out_features, in_features, out_f32, stream)
-                      : launch_wide<4, 4>(fn, x, weight, bias, y, rows, out_features, in_features, out_f32, stream);
+            return narrow ? launch_wide<2, 2>(fn, x, weight, bias, y, rows, out_features, in_features, out_f32, act, param, stream)
+                          : launch_wide<2, 4>(fn, x, weight, bias, y, rows, out_features, in_features, out_f32, act, param, stream);
+        return narrow ? launch_wide<4, 2>(fn, x, weight, bias, y, rows, out_features, in_features, out_f32, act, param, stream)
+                      : launch_wide<4, 4>(fn, x, weight, bias, y, rows, out_features, in_features, out_f32, act, param, stream);
     }
     const int64_t groups = cdiv(out_features, 16);
     const int waves = skinny_waves(groups, in_features);
@@ -140,9 +144,11 @@ extern "C" int nqh_skinny_linear(const void* x, const void* weight, const void* 
     const dim3 grid((unsigned)groups), block((unsigned)waves * 64);
     if (out_f32)
         skinny_linear_kernel<true><<<grid, block, lds, (hipStream_t)stream>>>(
-            (const uint16_t*)x, (const uint16_t*)weight, (const uint16_t*)bias, y, (int)rows, (int)out_features, (int)in_features);
+            (const uint16_t*)x, (const uint16_t*)weight, (const uint16_t*)bias, y, (int)rows, (int)out_features, (int)in_features, act,
+            param);
     else
         skinny_linear_kernel<false><<<grid, block, lds, (hipStream_t)stream>>>(
-            (const uint16_t*)x, (const uint16_t*)weight, (const uint16_t*)bias, y, (int)rows, (int)out_features, (int)in_features);
+            (const uint16_t*)x, (const uint16_t*)weight, (const uint16_t*)bias, y, (int)rows, (int)out_features, (int)in_features, act,
+            param);
     return launched(fn);
 }

@@ -141,6 +141,23 @@ __device__ __forceinline__ float decay_f32(float z, float inv_tau) {
     return __builtin_amdgcn_exp2f(-(l + fmaxf(-z, 0.f) * kLog2e_) * inv_tau);
 }
 
+// log(1 + e^z) = max(z, 0) + log(1 + e^-|z|), the logarithm as above.
+__device__ __forceinline__ float softplus_f32(float z) {
+    constexpr float kLog2e_ = 1.4426950408889634f, kLn2_ = 0.6931471805599453f;
+    const float x = __builtin_amdgcn_exp2f(-fabsf(z) * kLog2e_);
+    const float u = as_f32_result(1.f + x), um1 = as_f32_result(u - 1.f);
+    const float l = um1 == 0.f ? x : kLn2_ * __builtin_amdgcn_logf(u) * (x * __builtin_amdgcn_rcpf(um1));
+    return fmaxf(z, 0.f) + l;
+}
+// What may follow a matrix product (nqh_activation); param: the cap of NQH_ACT_SOFTCAP.
+__device__ __forceinline__ float activation_f32(float v, int act, float param) {
+    if (act == NQH_ACT_RELU2) {
+        v = fmaxf(v, 0.f);
+        return v * v;
+    }
+    return act == NQH_ACT_SOFTCAP ? param * tanhf(v / param) : v;
+}
+
 // ---- host-side error plumbing ---------------------------------------------------------------------
 int fail(int status, const char* fn, const char* fmt, ...);
 int launched(const char* fn);   // status of the launch just made

@@ -18,7 +18,7 @@ class Lease:
 class PagedKVCache:
     """Blocks of `block_size` tokens, [blocks, kv_heads, block_size, head_dim] per layer for K and V.  Uniform models
     hold all layers in one tensor ([layers, ...]); with `layer_shapes` -- (kv_heads, key row, value row) per layer run,
-    None for a run without attention -- every run has tensors of its own size, all of them indexed by the same block
+    None for a run without attention, a value row of 0 where keys and values share their row -- every run has tensors of its own size, all of them indexed by the same block
     numbers.  Rows may be wider than a head (padding stays zero: the writers never touch it)."""
 
     def __init__(self, num_layers: int, num_blocks: int, block_size: int, num_kv_heads: int = 0, head_dim: int = 0,
@@ -47,14 +47,16 @@ class PagedKVCache:
 
 
 class RecurrentStateCache:
-    """Recurrent state of `num_slots` sequences: fp32 [slots, heads, key dim, value dim] per layer run (`run_shapes`,
-    None for a run without state).  A slot is never cleared: the kernels take the state before position 0 as zero
+    """Recurrent state of `num_slots` sequences: fp32 [slots, *shape] per layer run (`run_shapes`, None for a run without
+    state), and for runs behind a short convolution the last inputs of that, `tail` [slots, *tail shape].  A slot is never cleared: the kernels take the state before position 0 as zero
     whatever the slot holds, so handing a slot on costs nothing and leaks nothing."""
 
-    def __init__(self, num_slots: int, run_shapes: Sequence[Optional[Tuple[int, int, int]]], device: "torch.device | str"):
+    def __init__(self, num_slots: int, run_shapes: Sequence[Optional[Tuple[int, ...]]], device: "torch.device | str",
+                 tail_shapes: Optional[Sequence[Optional[Tuple[int, ...]]]] = None):
         self.num_slots = num_slots
-        self.state = [None if s is None else torch.zeros(num_slots, *s, dtype=torch.float32, device=device)
-                      for s in run_shapes]
+        pool = lambda s: None if s is None else torch.zeros(num_slots, *s, dtype=torch.float32, device=device)
+        self.state = [pool(s) for s in run_shapes]
+        self.tail = [pool(s) for s in tail_shapes or [None] * len(self.state)]
         self.free: List[int] = list(range(num_slots - 1, -1, -1))
 
     def allocate(self) -> int:

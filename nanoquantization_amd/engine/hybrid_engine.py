@@ -1,25 +1,31 @@
 """Paged-KV and recurrent-state execution of HybridDecoder models (models/hybrid.py) on one MI355X.
 
-Residual stream.  fp32 throughout.  Every sublayer ends in a norm of its own and is followed by the next sublayer's
-norm, so one kernel (`residual_norm`) does both plus the addition -- and, in front of a repeated pass, adds the embedding
-output, gathered again from the table instead of being kept.
+Residual.  fp32 throughout, and written lazily: what a sublayer leaves is added by the kernel that also computes the next
+sublayer's norm.  `Residual` is one row per token; a sublayer may end in a norm of its own, and in front of a repeated pass the
+embedding output is added, gathered again from the table instead of being kept.  `Streams` are several rows per token under
+hyper-connections.
 
-Caches.  Every layer run (a looped layer runs several times) has its own K/V tensors, all indexed by the sequence's one
-block table, or its own state tensor, indexed by the sequence's state slot.  K/V rows are padded to a width the matrix-core
-kernels take.
+Caches.  Every layer run (a looped layer runs several times) has its own K/V tensors or its own latent rows, all indexed by
+the sequence's one block table, or its own state tensors, indexed by the sequence's state slot.  K/V and latent rows are padded
+to a width the matrix-core kernels take.
+
+Latent attention.  Decode steps and short portions take the queries into the latent space and attend to the latents
+themselves; longer prompt passes expand the contexts' latents to keys and values per head, which is fewer operations per
+query and key.
 
 Entry points.  `extend` runs any number of tokens of any number of sequences from where their caches stand (prompts,
 portions of prompts); `_decode_step` runs one token per batch row from the static buffers of EngineCore, in bf16 as a HIP
-graph of this library's kernels only.  Both share `_layers`."""
+graph of this library's kernels only.  Both share `_layers`; a `Step` tells the mixers which of the two is running."""
 from __future__ import annotations
 
 from dataclasses import dataclass
-from typing import Callable, Dict, List, Optional, Sequence
+from typing import Dict, List, Optional, Sequence
 
 import torch
 import torch.nn.functional as F
 
-from ..models.hybrid import AttentionSpec, GatedLinearSpec, HybridDecoder, RotarySpec, rotary_table
+from ..models.hybrid import (AttentionSpec, DenseSpec, GatedLinearSpec, HybridDecoder, LatentAttentionSpec, RotarySpec,
+                             SelectiveScanSpec, rotary_table)
 from . import hybrid_ops as ops
 from .cache import Lease, PagedKVCache, RecurrentStateCache
 from .core import EngineCore
@@ -34,8 +40,79 @@ class Portion:
     want: Sequence[int]
 
 
+@dataclass
+class Step:
+    """The tokens of one pass over the layers: a prompt pass has a layout, a decode step the tokens in each row's cache."""
+    ids: torch.Tensor
+    positions: torch.Tensor
+    slots: torch.Tensor
+    layout: Optional[ops.PromptPass] = None
+    context: Optional[torch.Tensor] = None
+
+
+class Residual:
+    """One fp32 row per token."""
+
+    def __init__(self, step: Step, table: torch.Tensor, eps: float, width: int):
+        self.eps, self.table, self.ids = eps, table, step.ids
+        self.x = torch.empty(step.ids.numel(), width, dtype=torch.float32, device=table.device)
+        self.pending: dict = dict(init=True, ids=step.ids, table=table)
+
+    def add_embedding(self) -> None:
+        self.pending.update(ids=self.ids, table=self.table)
+
+    def read(self, norm: torch.Tensor, hyper=None) -> torch.Tensor:
+        return ops.residual_norm(self.x, self.eps, next_weight=norm, **self.pending)
+
+    def read_routed(self, norm: torch.Tensor, router: torch.Tensor, top: int, ff: int):
+        return ops.residual_norm_route(self.x, self.eps, router, top, ff, norm, **self.pending)
+
+    def write(self, y: torch.Tensor, post_norm: Optional[torch.Tensor], hyper=None) -> None:
+        self.pending = dict(y=y, post_weight=post_norm)
+
+    def select(self, rows: torch.Tensor) -> None:
+        """Only these rows go on."""
+        self.x = self.x[rows].contiguous()
+        if "y" in self.pending:
+            self.pending["y"] = self.pending["y"][rows].contiguous()
+
+    def value(self) -> torch.Tensor:
+        if self.pending:
+            ops.residual_norm(self.x, self.eps, **self.pending)
+            self.pending = {}
+        return self.x.clone()
+
+
+class Streams:
+    """Several fp32 rows per token; `hyper` is the StreamWeights of the sublayer that reads or writes."""
+
+    def __init__(self, step: Step, table: torch.Tensor, eps: float, width: int, streams: int):
+        self.eps = eps
+        self.x = torch.empty(step.ids.numel(), streams, width, dtype=torch.float32, device=table.device)
+        self.pending: dict = dict(ids=step.ids, table=table)
+
+    def read(self, norm: torch.Tensor, hyper=None) -> torch.Tensor:
+        """`hyper` None: the plain sum of the streams."""
+        return ops.hyper_norm(self.x, self.eps, read=None if hyper is None else hyper.read, next_weight=norm, **self.pending)
+
+    def write(self, y: torch.Tensor, post_norm: Optional[torch.Tensor], hyper=None) -> None:
+        self.pending = dict(y=y, mix=hyper.mix, write=hyper.write)
+
+    def select(self, rows: torch.Tensor) -> None:
+        self.x = self.x[rows].contiguous()
+        if "y" in self.pending:
+            self.pending["y"] = self.pending["y"][rows].contiguous()
+
+    def value(self) -> torch.Tensor:
+        if self.pending:
+            ops.hyper_norm(self.x, self.eps, **self.pending)
+            self.pending = {}
+        return self.x.sum(dim=1)
+
+
 class HybridEngine(EngineCore):
     step_ops = ops
+    absorb_rows = ops.SKINNY_ROWS       # prompt passes of up to so many rows attend to latents as a decode step does
 
     def __init__(self, model: HybridDecoder, max_batch: int, max_seq_len: int, block_size: int = 64,
                  num_blocks: Optional[int] = None, use_graph: bool = True, num_slots: Optional[int] = None,
@@ -45,76 +122,145 @@ class HybridEngine(EngineCore):
         self.spec = spec = model.spec
         # a graph may hold this library's kernels only: products in fp32, of odd widths or of many rows are the vendor
         # library's, which may record memory-clearing nodes
-        linears = [model.head] + [w for l in model.layers
-                                  for w in (l.mixer.out, l.mixer.qkv if hasattr(l.mixer, "qkv") else l.mixer.proj)]
+        linears = [model.head] + [w for l in model.layers for w in l.linears()]
         super().__init__(p.device, p.dtype, max_batch, max_seq_len, block_size, num_blocks,
                          use_graph and all(ops.skinny_linear_supported(max_batch, w) for w in linears))
         self.runs = spec.runs()
         self.prefill_tokens = prefill_tokens
         mixers = [spec.layers[i].mixer for i, _ in self.runs]
-        self.cache = PagedKVCache(len(mixers), self.num_blocks, block_size, dtype=self.dtype, device=self.device, layer_shapes=[
-            (m.kv_heads, *ops.cache_rows(m.dim, m.vdim, self.dtype)) if isinstance(m, AttentionSpec) else None for m in mixers])
-        state_shapes = [(m.heads, m.dim, m.vdim) if isinstance(m, GatedLinearSpec) else None for m in mixers]
+        self.cache = PagedKVCache(len(mixers), self.num_blocks, block_size, dtype=self.dtype, device=self.device,
+                                  layer_shapes=[self._cache_shape(m) for m in mixers])
+        state_shapes, tail_shapes = zip(*(self._state_shapes(m) for m in mixers))
         if any(state_shapes):
-            self.states = RecurrentStateCache(num_slots or max_batch, state_shapes, self.device)
+            self.states = RecurrentStateCache(num_slots or max_batch, state_shapes, self.device, tail_shapes)
         self._angles: Dict[RotarySpec, torch.Tensor] = {}
-        for m in mixers:
-            if isinstance(m, AttentionSpec) and m.rotary is not None and m.rotary not in self._angles:
-                self._angles[m.rotary] = rotary_table(m.rotary, self.max_ctx).to(self.device)
+        for rot in (getattr(m, "rotary", None) for m in mixers):
+            if rot is not None and rot not in self._angles:
+                self._angles[rot] = rotary_table(rot, self.max_ctx).to(self.device)
+        # latent attention: the expansions per head, as the products into and out of the latent space want them
+        self._per_head = {i: model.layers[i].mixer.per_head() for i, l in enumerate(spec.layers)
+                          if isinstance(l.mixer, LatentAttentionSpec)}
+
+    def _cache_shape(self, m):
+        if isinstance(m, AttentionSpec):
+            return (m.kv_heads, *ops.cache_rows(m.dim, m.vdim, self.dtype))
+        if isinstance(m, LatentAttentionSpec):
+            return (1, ops.latent_row(m.rank, m.rotary.dims, self.dtype)[1], 0)
+        return None
+
+    @staticmethod
+    def _state_shapes(m):
+        """(recurrent state, last inputs of the convolution) of a run; None: has none."""
+        if isinstance(m, GatedLinearSpec):
+            return (m.heads, m.dim, m.vdim), None
+        if isinstance(m, SelectiveScanSpec):
+            return (m.state, m.channels), (m.taps - 1, m.channels)
+        return None, None
 
     # ---- pieces shared by prefill and decode ---------------------------------------------------------
-    def _linear(self, x: torch.Tensor, w: torch.Tensor, b: Optional[torch.Tensor] = None) -> torch.Tensor:
+    def _linear(self, x: torch.Tensor, w: torch.Tensor, b: Optional[torch.Tensor] = None, activation: Optional[str] = None,
+                param: float = 0.0) -> torch.Tensor:
         if ops.skinny_linear_supported(x.shape[0], w):
-            return ops.skinny_linear(x, w, b)
-        return F.linear(x, w, b)
+            return ops.skinny_linear(x, w, b, activation=activation, param=param)
+        y = F.linear(x, w, b)
+        return y if activation is None else ops.activate_(y, activation, param)
 
     def _logits(self, h: torch.Tensor) -> torch.Tensor:
         """fp32 logits of normalised rows."""
-        w = self.model.head
-        if h.dtype == torch.float32:
-            return F.linear(h, w)
-        if not ops.skinny_linear_supported(1, w):
-            return F.linear(h, w).float()
-        parts = [ops.skinny_linear(p, w, out_f32=True) for p in h.split(ops.SKINNY_ROWS)]
-        return parts[0] if len(parts) == 1 else torch.cat(parts)
+        w, cap = self.model.head, self.spec.logit_cap
+        act = "softcap" if cap else None
+        if h.dtype != torch.float32 and ops.skinny_linear_supported(1, w):
+            parts = [ops.skinny_linear(p, w, out_f32=True, activation=act, param=cap) for p in h.split(ops.SKINNY_ROWS)]
+            return parts[0] if len(parts) == 1 else torch.cat(parts)
+        y = F.linear(h, w).float()
+        return ops.activate_(y, act, cap) if act else y
 
-    def _layers(self, ids: torch.Tensor, positions: torch.Tensor, slots: torch.Tensor, attend: Callable, recur: Callable,
-                rows: Optional[torch.Tensor] = None, trace: Optional[list] = None) -> torch.Tensor:
-        """All layer runs for the given tokens; returns the final norm of the residual rows `rows` (all if None).
-        attend(run, spec, q) and recur(run, spec, weights, proj) supply the mixers' access to cache and state.
-        `trace` receives the residual stream after every run (costs extra launches)."""
-        model, eps = self.model, self.spec.eps
-        x = torch.empty(ids.numel(), self.spec.width, dtype=torch.float32, device=self.device)
-        pending: dict = dict(init=True, ids=ids, table=model.embed)
+    # ---- mixers: h [rows, width] -> what the output projection takes ------------------------------------
+    def _attention(self, run: int, m: AttentionSpec, w, h: torch.Tensor, step: Step) -> torch.Tensor:
+        k, v = self.cache.k[run], self.cache.v[run]
+        cos_sin = self._angles[m.rotary] if m.rotary is not None else None
+        q = ops.qk_norm_rope_store(self._linear(h, w.qkv, w.qkv_bias), w.q_norm, w.k_norm, cos_sin, step.positions, step.slots,
+                                   k, v, m.heads, m.dim, m.vdim, self.spec.eps)
+        if step.layout is not None:
+            return ops.attention_prefill(q, k, v, step.layout, m.dim, m.vdim, m.scale, m.chunk, m.window, w.sink)
+        return ops.attention_decode(q, k, v, self.s_table, step.context, m.dim, m.vdim, m.scale, m.chunk, m.window, w.sink)
+
+    def _latent_attention(self, run: int, m: LatentAttentionSpec, w, h: torch.Tensor, step: Step) -> torch.Tensor:
+        cache, rot, eps = self.cache.k[run], m.rotary.dims, self.spec.eps
+        rot_at, row = ops.latent_row(m.rank, rot, self.dtype)
+        proj, cos_sin, rows = self._linear(h, w.proj), self._angles[m.rotary], h.shape[0]
+        wide = 0
+        if step.layout is not None and rows > self.absorb_rows:
+            wide = ops.latent_prefill_query_row(m.dim, rot, m.vdim, m.rank, self.dtype)
+        if wide:
+            q = ops.latent_store(proj, w.latent_norm, cos_sin, step.positions, step.slots, cache, m.heads, m.dim, rot_at, eps,
+                                 wide, m.dim, True)
+            latents = ops.latent_gather(cache, step.layout, m.rank, rot, rot_at)
+            return ops.latent_attention_prefill(q, F.linear(latents[:, :m.rank], w.expand), latents[:, m.rank:], step.layout,
+                                                m.dim, m.vdim, m.scale)
+        into, out_of = self._per_head[self.runs[run][0]]
+        q = ops.latent_store(proj, w.latent_norm, cos_sin, step.positions, step.slots, cache, m.heads, m.dim, rot_at, eps, row,
+                             rot_at, False)
+        ops.head_linear(proj[:, :w.splits[0]].view(rows, m.heads, m.dim + rot), into, q)
+        if step.layout is None:
+            o = ops.latent_attention_decode(q, cache, self.s_table, step.context, m.rank, rot_at, m.scale)
+        elif rows <= self.absorb_rows:
+            o = ops.latent_attention_decode(q, cache, *step.layout.row_tables(), m.rank, rot_at, m.scale)
+        else:       # the latent row as key and as value of a single head
+            o = ops.attention_prefill(q, cache, cache, step.layout, row, m.rank, m.scale).view(rows, m.heads, m.rank)
+        return ops.head_linear(o, out_of, torch.empty(rows, m.heads, m.vdim, dtype=o.dtype, device=o.device)).view(rows, -1)
+
+    def _gated_linear(self, run: int, m: GatedLinearSpec, w, h: torch.Tensor, step: Step) -> torch.Tensor:
+        proj, state = self._linear(h, w.proj), self.states.state[run]
+        if step.layout is None:
+            return ops.gla_decode(proj, w.decay_up, w.decay_bias, w.head_norm, state, self.s_slot, self.s_pos, self.s_active,
+                                  m.heads, m.dim, m.vdim, m.tau, self.spec.eps)
+        decay = ops.gla_decay(proj, w.decay_up, w.decay_bias, m.heads, m.dim, m.vdim, m.tau)
+        o = ops.gla_prefill(proj, decay, state, step.layout, m.heads, m.dim, m.vdim, m.rank)
+        return ops.head_norm_gate(o, proj, w.head_norm, m.heads, m.dim, m.vdim, m.rank, self.spec.eps)
+
+    def _selective_scan(self, run: int, m: SelectiveScanSpec, w, h: torch.Tensor, step: Step) -> torch.Tensor:
+        state, tail = self.states.state[run], self.states.tail[run]
+        x_in, z = self._linear(h, w.proj).split([m.channels, m.channels], dim=1)
+        if step.layout is None:
+            x = ops.conv_step(x_in, w.conv, w.conv_bias, tail, self.s_slot, self.s_pos, self.s_active)
+        else:
+            piece = ops.scan_piece_rows(h.shape[0], m.channels, m.state)
+            x = ops.conv_silu(x_in, w.conv, w.conv_bias, tail, step.layout, piece)
+        low, bc = self._linear(x, w.select).split([m.dt_rank, 2 * m.state], dim=1)
+        dt = ops.scan_dt(low, w.dt_up, w.dt_bias)
+        if step.layout is None:
+            return ops.scan_step(x, dt, bc, z, w.a_log, w.skip, state, self.s_slot, self.s_pos, self.s_active)
+        return ops.scan_prefill(x, dt, bc, z, w.a_log, w.skip, x_in, state, tail, step.layout, piece)
+
+    _MIXERS = {AttentionSpec: _attention, LatentAttentionSpec: _latent_attention, GatedLinearSpec: _gated_linear,
+               SelectiveScanSpec: _selective_scan}
+
+    def _layers(self, step: Step, rows: Optional[torch.Tensor] = None, trace: Optional[list] = None) -> torch.Tensor:
+        """All layer runs for the given tokens; returns the final norm of the residual rows `rows` (all if None).  `trace`
+        receives the residual (the sum of its streams) after every run (costs extra launches)."""
+        model, spec = self.model, self.spec
+        args = (step, model.embed, spec.eps, spec.width)
+        res = Streams(*args, spec.streams) if spec.streams else Residual(*args)
         for run, (li, add_embedding) in enumerate(self.runs):
-            layer, spec = model.layers[li], self.spec.layers[li]
+            layer, ls = model.layers[li], spec.layers[li]
             if add_embedding:
-                pending.update(ids=ids, table=model.embed)
-            h = ops.residual_norm(x, eps, next_weight=layer.norm_mixer, **pending)
-            mix, m = layer.mixer, spec.mixer
-            if isinstance(m, AttentionSpec):
-                cos_sin = self._angles[m.rotary] if m.rotary is not None else None
-                q = ops.qk_norm_rope_store(self._linear(h, mix.qkv, mix.qkv_bias), mix.q_norm, mix.k_norm, cos_sin,
-                                           positions, slots, self.cache.k[run], self.cache.v[run], m.heads, m.dim, m.vdim,
-                                           eps)
-                o = attend(run, m, q)
-            else:
-                o = recur(run, m, mix, self._linear(h, mix.proj))
-            pending = dict(y=self._linear(o, mix.out), post_weight=layer.norm_mixer_out)
-            if spec.mlp is not None:
-                h, routing = ops.residual_norm_route(x, eps, layer.mlp.router, spec.mlp.top, spec.mlp.ff, layer.norm_mlp,
-                                                     **pending)
-                pending = dict(y=ops.moe_experts(h, layer.mlp.gate_up, layer.mlp.down, routing),
-                               post_weight=layer.norm_mlp_out)
+                res.add_embedding()
+            h = res.read(layer.norm_mixer, layer.mixer_streams)
+            o = self._MIXERS[type(ls.mixer)](self, run, ls.mixer, layer.mixer, h, step)
+            res.write(self._linear(o, layer.mixer.out), layer.norm_mixer_out, layer.mixer_streams)
+            if isinstance(ls.mlp, DenseSpec):
+                h = res.read(layer.norm_mlp, layer.mlp_streams)
+                y = self._linear(self._linear(h, layer.mlp.up, activation=ls.mlp.activation), layer.mlp.down)
+                res.write(y, layer.norm_mlp_out, layer.mlp_streams)
+            elif ls.mlp is not None:
+                h, routing = res.read_routed(layer.norm_mlp, layer.mlp.router, ls.mlp.top, ls.mlp.ff)
+                res.write(ops.moe_experts(h, layer.mlp.gate_up, layer.mlp.down, routing), layer.norm_mlp_out)
             if trace is not None:
-                ops.residual_norm(x, eps, **pending)
-                trace.append(x.clone())
-                pending = {}
+                trace.append(res.value())
         if rows is not None:
-            x = x[rows].contiguous()
-            if pending:
-                pending["y"] = pending["y"][rows].contiguous()
-        return ops.residual_norm(x, eps, next_weight=model.final_norm, **pending)
+            res.select(rows)
+        return res.read(model.final_norm)
 
     # ---- any number of tokens of any number of sequences ------------------------------------------------
     @torch.no_grad()
@@ -140,19 +286,12 @@ class HybridEngine(EngineCore):
         packed = torch.tensor([ids, pos, slots], dtype=torch.long).to(dev)
         ids_d, pos_d, slots_d = packed[0], packed[1], packed[2]
 
-        def attend(run, m, q):
-            return ops.attention_prefill(q, self.cache.k[run], self.cache.v[run], layout, m.dim, m.vdim, m.scale, m.chunk)
-
-        def recur(run, m, w, proj):
-            decay = ops.gla_decay(proj, w.decay_up, w.decay_bias, m.heads, m.dim, m.vdim, m.tau)
-            o = ops.gla_prefill(proj, decay, self.states.state[run], layout, m.heads, m.dim, m.vdim, m.rank)
-            return ops.head_norm_gate(o, proj, w.head_norm, m.heads, m.dim, m.vdim, m.rank, self.spec.eps)
-
+        step = Step(ids_d, pos_d, slots_d, layout=layout)
         rows = torch.tensor(want, dtype=torch.long).to(dev)
         if not want:        # the pass still fills cache and state
-            self._layers(ids_d, pos_d, slots_d, attend, recur, trace=trace)
+            self._layers(step, trace=trace)
             return torch.empty(0, self.spec.vocab, dtype=torch.float32, device=dev)
-        return self._logits(self._layers(ids_d, pos_d, slots_d, attend, recur, rows, trace))
+        return self._logits(self._layers(step, rows, trace))
 
     def _prefill_ragged(self, prompts: List[List[int]], leases: List[Lease]) -> torch.Tensor:
         """Whole prompts; longer ones than `prefill_tokens` in portions, the rest of the pass filled with the next."""
@@ -190,13 +329,4 @@ class HybridEngine(EngineCore):
     # ---- one token per batch row -----------------------------------------------------------------------
     def _decode_step(self) -> None:
         slots, ctx = ops.decode_prepare(self.s_pos, self.s_active, self.s_table, self.block_size)
-
-        def attend(run, m, q):
-            return ops.attention_decode(q, self.cache.k[run], self.cache.v[run], self.s_table, ctx, m.dim, m.vdim, m.scale,
-                                        m.chunk)
-
-        def recur(run, m, w, proj):
-            return ops.gla_decode(proj, w.decay_up, w.decay_bias, w.head_norm, self.states.state[run], self.s_slot,
-                                  self.s_pos, self.s_active, m.heads, m.dim, m.vdim, m.tau, self.spec.eps)
-
-        self._finish_step(self._logits(self._layers(self.s_ids, self.s_pos, slots, attend, recur)))
+        self._finish_step(self._logits(self._layers(Step(self.s_ids, self.s_pos, slots, context=ctx))))

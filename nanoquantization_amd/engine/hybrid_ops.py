@@ -12,7 +12,7 @@ from .. import _lib
 
 _DTYPES = {torch.bfloat16: 1, torch.float32: 2}
 SKINNY_ROWS = 64
-
+ACTIVATIONS = {None: 0, "relu2": 1, "softcap": 2}      # what may follow a product; "softcap" takes the cap as parameter
 
 _MATRIX_ROWS = (32, 64, 96, 128, 192, 256)      # cache row widths the matrix-core attention kernels exist for
 
@@ -26,6 +26,15 @@ def cache_rows(dim: int, vdim: int, dtype: torch.dtype) -> Tuple[int, int]:
         if max(dim, vdim) <= row:
             return row, row
     return (dim + 31) // 32 * 32, (vdim + 31) // 32 * 32
+
+
+def latent_row(rank: int, rot_dim: int, dtype: torch.dtype) -> Tuple[int, int]:
+    """(place of the rotated part, width) of a latent cache row: in bf16 padded to what the matrix-core kernel takes, in
+    fp32 and beyond its sizes without padding."""
+    if dtype == torch.bfloat16 and rank <= 512 and rot_dim <= 64:
+        at = next(r for r in (64, 128, 256, 512) if rank <= r)
+        return at, at + (32 if rot_dim <= 32 else 64)
+    return rank, rank + rot_dim
 
 
 def _dtype(t: torch.Tensor) -> int:
@@ -83,6 +92,34 @@ def residual_norm(x: torch.Tensor, eps: float, *, y: Optional[torch.Tensor] = No
     dev, h, dt, args = _residual_args(x, eps, y, post_weight, ids, table, init, next_weight, dtype)
     _call(dev, "nqh_residual_norm", *args, *x.shape, eps, _DTYPES[dt])
     return h
+
+
+def hyper_norm(x: torch.Tensor, eps: float, *, ids: Optional[torch.Tensor] = None, table: Optional[torch.Tensor] = None,
+               y: Optional[torch.Tensor] = None, mix: Optional[torch.Tensor] = None, write: Optional[torch.Tensor] = None,
+               read: Optional[torch.Tensor] = None, next_weight: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """The fp32 residual streams x [rows, streams, width] IN PLACE: all set to table[ids], or mixed anew from the old ones
+    and a sublayer's output y; returns RMSNorm(sum of the streams times read, or of the streams as they are) * next_weight
+    (None without next_weight)."""
+    dev = _dev(x, ids, table, y, mix, write, read, next_weight)
+    rows, streams, width = x.shape
+    assert x.dtype == torch.float32
+    operands = [t for t in (table, y, mix, write, read, next_weight) if t is not None]
+    dt = operands[0].dtype
+    assert all(t.dtype == dt for t in operands)
+    assert ids is None or (y is None and ids.dtype == torch.int64 and ids.numel() == rows and table.shape[1] == width)
+    assert y is None or (y.shape == (rows, width) and mix.shape == (streams, streams) and write.shape == (streams,))
+    assert read is None or read.shape == (streams,)
+    assert next_weight is None or next_weight.shape == (width,)
+    h = torch.empty(rows, width, dtype=dt, device=dev) if next_weight is not None else None
+    _call(dev, "nqh_hyper_norm", x.data_ptr(), _ptr(ids), _ptr(table), 0 if table is None else table.shape[0], _ptr(y),
+          _ptr(mix), _ptr(write), _ptr(read), _ptr(next_weight), _ptr(h), rows, streams, width, eps, _DTYPES[dt])
+    return h
+
+
+def activate_(x: torch.Tensor, activation: str, param: float = 0.0) -> torch.Tensor:
+    """activation(x) IN PLACE."""
+    _call(_dev(x), "nqh_activate", x.data_ptr(), x.numel(), ACTIVATIONS[activation], param, _dtype(x))
+    return x
 
 
 class Routing:
@@ -180,11 +217,29 @@ class PromptPass:
         self.num_tiles, self.max_blocks = len(tiles), width
         packed = torch.tensor(table + seg + flat, dtype=torch.int32).to(device)
         self.tables, self.seg, self.tiles = packed.split([len(table), len(seg), len(flat)])
-        self._pieces = {}
+        self._pieces, self._contexts, self._row_tables = {}, None, None
 
-    def pieces(self, heads: int, dim: int, vdim: int) -> Tuple[torch.Tensor, int, bool]:
-        """(piece list for gla_prefill, its length, whether a sequence has several) for a head size."""
-        size = _lib.hybrid_lib().nqh_gla_piece_rows(self.rows, heads, dim, vdim)
+    def contexts(self) -> Tuple[torch.Tensor, int, int]:
+        """The segments' contexts laid out one after the other: (first row of each, int32; rows in all; the longest)."""
+        if self._contexts is None:
+            lens = [start + rows for start, rows, _, _ in self.segments]
+            first = [sum(lens[:i]) for i in range(len(lens))]
+            self._contexts = torch.tensor(first, dtype=torch.int32).to(self.device), sum(lens), max(lens)
+        return self._contexts
+
+    def row_tables(self) -> Tuple[torch.Tensor, torch.Tensor]:
+        """The pass as a decode step sees it, every token a row of its own: (block tables [rows, max_blocks], tokens in the
+        cache up to and including it [rows])."""
+        if self._row_tables is None:
+            seg = [i for i, s in enumerate(self.segments) for _ in range(s[1])]
+            ctx = [s[0] + t + 1 for s in self.segments for t in range(s[1])]
+            seg, ctx = torch.tensor([seg, ctx], dtype=torch.int32).to(self.device)
+            self._row_tables = self.tables.view(len(self.segments), self.max_blocks)[seg.long()].contiguous(), ctx.contiguous()
+        return self._row_tables
+
+    def pieces(self, size: int) -> Tuple[torch.Tensor, int, bool]:
+        """(list of pieces of at most `size` rows for gla_prefill and scan_prefill, its length, whether a sequence has
+        several)."""
         if size not in self._pieces:
             out, first, chained = [], 0, False
             for start, rows, _, slot in self.segments:
@@ -198,37 +253,238 @@ class PromptPass:
 
 
 def attention_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, layout: PromptPass, dim: int, vdim: int,
-                      scale: float, chunk: int = 0) -> torch.Tensor:
+                      scale: float, chunk: int = 0, window: int = 0, sink: Optional[torch.Tensor] = None) -> torch.Tensor:
     """q [rows, heads, k row]: the tokens of the pass, attending to their sequences' caches (their own keys are already
-    there).  chunk > 0: only keys of the query's own chunk of that many positions.  Returns [rows, heads * vdim]."""
+    there).  chunk > 0: only keys of the query's own chunk of that many positions; window > 0: only the query's own and the
+    window - 1 positions before it.  sink [heads]: a further unscaled score per head, without key or value.  Returns
+    [rows, heads * vdim]."""
     rows, heads = q.shape[:2]
-    dev = _dev(q, k_cache, v_cache, layout.tables)
+    dev = _dev(q, k_cache, v_cache, sink, layout.tables)
+    assert sink is None or (sink.shape == (heads,) and sink.dtype == q.dtype)
     blocks, kv_heads, block_size, k_row, v_row = _check_attention(q, k_cache, v_cache, heads)
     assert rows == layout.rows
     out = torch.empty(rows, heads * vdim, dtype=q.dtype, device=dev)
     _call(dev, "nqh_attention_prefill", q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), layout.tables.data_ptr(),
-          layout.seg.data_ptr(), layout.tiles.data_ptr(), out.data_ptr(), rows, layout.num_tiles, heads, kv_heads, dim, vdim,
-          k_row, v_row, block_size, layout.max_blocks, blocks, chunk, scale, _dtype(q))
+          layout.seg.data_ptr(), layout.tiles.data_ptr(), _ptr(sink), out.data_ptr(), rows, layout.num_tiles, heads, kv_heads,
+          dim, vdim, k_row, v_row, block_size, layout.max_blocks, blocks, chunk, window, scale, _dtype(q))
     return out
 
 
 def attention_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
-                     context_lens: torch.Tensor, dim: int, vdim: int, scale: float, chunk: int = 0) -> torch.Tensor:
+                     context_lens: torch.Tensor, dim: int, vdim: int, scale: float, chunk: int = 0, window: int = 0,
+                     sink: Optional[torch.Tensor] = None) -> torch.Tensor:
     """One query token per sequence, the last of its context_lens [batch] int32 cached tokens; block_table int32
     [batch, max_blocks].  Returns [batch, heads * vdim]."""
     batch, heads = q.shape[:2]
-    dev = _dev(q, k_cache, v_cache, block_table, context_lens)
+    dev = _dev(q, k_cache, v_cache, block_table, context_lens, sink)
+    assert sink is None or (sink.shape == (heads,) and sink.dtype == q.dtype)
     blocks, kv_heads, block_size, k_row, v_row = _check_attention(q, k_cache, v_cache, heads)
     assert block_table.dtype == torch.int32 and block_table.dim() == 2 and block_table.shape[0] == batch
     assert context_lens.dtype == torch.int32 and context_lens.shape == (batch,)
     max_blocks = block_table.shape[1]
     out = torch.empty(batch, heads * vdim, dtype=q.dtype, device=dev)
     nbytes = _lib.hybrid_lib().nqh_attention_decode_workspace_bytes(batch, heads, kv_heads, v_row, block_size * max_blocks,
-                                                                    chunk, _dtype(q))
+                                                                    chunk, window, _dtype(q))
     ws = torch.empty(nbytes, dtype=torch.uint8, device=dev) if nbytes else None
     _call(dev, "nqh_attention_decode", q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), block_table.data_ptr(),
-          context_lens.data_ptr(), out.data_ptr(), batch, heads, kv_heads, dim, vdim, k_row, v_row, block_size, max_blocks,
-          blocks, chunk, scale, _dtype(q), _ptr(ws), nbytes)
+          context_lens.data_ptr(), _ptr(sink), out.data_ptr(), batch, heads, kv_heads, dim, vdim, k_row, v_row, block_size,
+          max_blocks, blocks, chunk, window, scale, _dtype(q), _ptr(ws), nbytes)
+    return out
+
+
+# ---- latent attention --------------------------------------------------------------------------------------------------
+def latent_store(proj: torch.Tensor, norm_weight: torch.Tensor, cos_sin: torch.Tensor, positions: torch.Tensor,
+                 slots: torch.Tensor, cache: torch.Tensor, heads: int, dim: int, rot_at: int, eps: float, q_row: int,
+                 rot_q: int, copy_plain: bool) -> torch.Tensor:
+    """proj [rows, heads * (dim + rot) + rank + rot]: the latent normalised and the shared key part rotated into their cache
+    rows [blocks, 1, block_size, row]; returns q [rows, heads, q_row] with the rotated part at rot_q and, if copy_plain, the
+    unrotated one in front (else that place is left to head_linear)."""
+    dev = _dev(proj, norm_weight, cos_sin, positions, slots, cache)
+    rows, rot_dim, rank = proj.shape[0], cos_sin.shape[1], norm_weight.shape[0]
+    blocks, one, block_size, row = cache.shape
+    assert one == 1 and proj.shape[1] == heads * (dim + rot_dim) + rank + rot_dim
+    assert norm_weight.dtype == proj.dtype and cache.dtype == proj.dtype and cos_sin.dtype == torch.float32
+    assert positions.dtype == torch.int64 and slots.dtype == torch.int64
+    assert positions.numel() == rows and slots.numel() == rows
+    q = torch.empty(rows, heads, q_row, dtype=proj.dtype, device=dev)
+    _call(dev, "nqh_latent_store", proj.data_ptr(), norm_weight.data_ptr(), cos_sin.data_ptr(), positions.data_ptr(),
+          slots.data_ptr(), q.data_ptr(), cache.data_ptr(), rows, heads, dim, rot_dim, rank, q_row, rot_q, int(copy_plain),
+          row, rot_at, cos_sin.shape[0], blocks * block_size, eps, _dtype(proj))
+    return q
+
+
+def head_linear(x: torch.Tensor, weight: torch.Tensor, y: torch.Tensor) -> torch.Tensor:
+    """y[r, h, :out] = weight[h] x[r, h, :in] for weight [heads, out, in]; x and y are 3-d, last dimension dense, and may be
+    views."""
+    heads, n_out, n_in = weight.shape
+    dev = _dev(weight)
+    assert x.device == dev and y.device == dev and x.dtype == weight.dtype and y.dtype == weight.dtype
+    rows = x.shape[0]
+    assert x.shape[1] == heads and x.shape[2] >= n_in and y.shape[:2] == (rows, heads) and y.shape[2] >= n_out
+    assert x.stride(2) == 1 and y.stride(2) == 1
+    _call(dev, "nqh_head_linear", x.data_ptr(), weight.data_ptr(), y.data_ptr(), rows, heads, n_out, n_in, x.stride(0),
+          x.stride(1), y.stride(0), y.stride(1), _dtype(weight))
+    return y
+
+
+def latent_prefill_query_row(dim: int, rot_dim: int, vdim: int, rank: int, dtype: torch.dtype) -> int:
+    """Width of a query row for latent_prefill_expanded; 0 if it does not take these sizes."""
+    if dtype not in _DTYPES or rank % 8:
+        return 0
+    return _lib.hybrid_lib().nqh_latent_attention_prefill_query_row(dim, rot_dim, vdim, _DTYPES[dtype])
+
+
+def latent_gather(cache: torch.Tensor, layout: PromptPass, rank: int, rot_dim: int, rot_at: int) -> torch.Tensor:
+    """[rows of all contexts, rank + rot_dim]: the cached rows of the segments' contexts without their padding."""
+    dev = _dev(cache, layout.tables)
+    first, total, longest = layout.contexts()
+    blocks, _, block_size, row = cache.shape
+    assert cache.element_size() == 2
+    out = torch.empty(total, rank + rot_dim, dtype=cache.dtype, device=dev)
+    _call(dev, "nqh_latent_gather", cache.data_ptr(), layout.tables.data_ptr(), layout.seg.data_ptr(), first.data_ptr(),
+          out.data_ptr(), len(layout.segments), longest, rank, rot_dim, row, rot_at, block_size, layout.max_blocks, blocks)
+    return out
+
+
+def latent_attention_prefill(q: torch.Tensor, kv: torch.Tensor, rot: torch.Tensor, layout: PromptPass, dim: int, vdim: int,
+                             scale: float) -> torch.Tensor:
+    """q [rows, heads, latent_prefill_query_row]; kv [context rows, heads * (dim + vdim)] and rot [context rows, rot] (a view
+    with dense rows is enough) of the contexts as `latent_gather` lays them out.  Returns [rows, heads * vdim]."""
+    dev = _dev(q, layout.tables)
+    rows, heads = q.shape[:2]
+    first, total, _ = layout.contexts()
+    assert rows == layout.rows and kv.shape == (total, heads * (dim + vdim)) and rot.shape[0] == total
+    assert kv.dtype == q.dtype == rot.dtype == torch.bfloat16 and kv.stride(1) == 1 and rot.stride(1) == 1
+    assert q.shape[2] == _lib.hybrid_lib().nqh_latent_attention_prefill_query_row(dim, rot.shape[1], vdim, _dtype(q))
+    out = torch.empty(rows, heads * vdim, dtype=q.dtype, device=dev)
+    _call(dev, "nqh_latent_attention_prefill", q.data_ptr(), kv.data_ptr(), kv.stride(0), rot.data_ptr(), rot.stride(0),
+          first.data_ptr(), layout.seg.data_ptr(), layout.tiles.data_ptr(), out.data_ptr(), rows, layout.num_tiles, heads,
+          dim, rot.shape[1], vdim, scale)
+    return out
+
+
+def latent_attention_decode(q: torch.Tensor, cache: torch.Tensor, block_table: torch.Tensor, context_lens: torch.Tensor,
+                            rank: int, rot_at: int, scale: float) -> torch.Tensor:
+    """One query token per row, q [batch, heads, row] in the latent space; returns [batch, heads, rank] in it."""
+    dev = _dev(q, cache, block_table, context_lens)
+    batch, heads, row = q.shape
+    blocks, one, block_size, width = cache.shape
+    assert one == 1 and width == row and cache.dtype == q.dtype
+    assert block_table.dtype == torch.int32 and block_table.dim() == 2 and block_table.shape[0] == batch
+    assert context_lens.dtype == torch.int32 and context_lens.shape == (batch,)
+    max_blocks = block_table.shape[1]
+    out = torch.empty(batch, heads, rank, dtype=q.dtype, device=dev)
+    nbytes = _lib.hybrid_lib().nqh_latent_attention_decode_workspace_bytes(batch, heads, rank, rot_at, row,
+                                                                           block_size * max_blocks, _dtype(q))
+    ws = torch.empty(nbytes, dtype=torch.uint8, device=dev) if nbytes else None
+    _call(dev, "nqh_latent_attention_decode", q.data_ptr(), cache.data_ptr(), block_table.data_ptr(), context_lens.data_ptr(),
+          out.data_ptr(), batch, heads, rank, rot_at, row, block_size, max_blocks, blocks, scale, _dtype(q), _ptr(ws), nbytes)
+    return out
+
+
+# ---- selective scan ------------------------------------------------------------------------------------------------------
+def scan_piece_rows(rows: int, channels: int, states: int) -> int:
+    return _lib.hybrid_lib().nqh_scan_piece_rows(rows, channels, states)
+
+
+def _rows_of(t: torch.Tensor, dev: torch.device, width: int) -> None:
+    """t is a view of `width` columns with dense rows."""
+    assert t.device == dev and t.dim() == 2 and t.shape[1] == width and t.stride(1) == 1
+
+
+def conv_silu(x: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor, tail: torch.Tensor, layout: PromptPass,
+              piece_rows: int) -> torch.Tensor:
+    """silu(causal convolution per channel + bias) of the pass's rows x [rows, channels] (a view); `tail` [slots, taps - 1,
+    channels] supplies the inputs ahead of a portion and is left as it is (scan_prefill moves it on)."""
+    dev = _dev(weight, bias, tail, layout.tables)
+    channels, taps = weight.shape
+    _rows_of(x, dev, channels)
+    assert x.shape[0] == layout.rows and bias.shape == (channels,) and weight.dtype == bias.dtype == x.dtype
+    assert tail.dtype == torch.float32 and tail.shape[1:] == (taps - 1, channels)
+    assert all(0 <= s[3] < tail.shape[0] for s in layout.segments)
+    pieces, n, _ = layout.pieces(piece_rows)
+    out = torch.empty(layout.rows, channels, dtype=x.dtype, device=dev)
+    _call(dev, "nqh_conv_silu", x.data_ptr(), x.stride(0), weight.data_ptr(), bias.data_ptr(), tail.data_ptr() or None,
+          pieces.data_ptr(), n, min(piece_rows, max(s[1] for s in layout.segments)), out.data_ptr(), channels, taps, _dtype(x))
+    return out
+
+
+def conv_step(x: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor, tail: torch.Tensor, slots: torch.Tensor,
+              positions: torch.Tensor, active: torch.Tensor) -> torch.Tensor:
+    """The same for one token per sequence; `tail` is moved on IN PLACE at the rows' slots."""
+    dev = _dev(weight, bias, tail, slots, positions, active)
+    channels, taps = weight.shape
+    _rows_of(x, dev, channels)
+    batch = x.shape[0]
+    assert bias.shape == (channels,) and weight.dtype == bias.dtype == x.dtype
+    assert tail.dtype == torch.float32 and tail.shape[1:] == (taps - 1, channels)
+    assert slots.dtype == torch.int32 and positions.dtype == torch.int64 and active.dtype == torch.bool
+    assert slots.numel() == batch and positions.numel() == batch and active.numel() == batch
+    out = torch.empty(batch, channels, dtype=x.dtype, device=dev)
+    _call(dev, "nqh_conv_step", x.data_ptr(), x.stride(0), weight.data_ptr(), bias.data_ptr(), tail.data_ptr() or None,
+          slots.data_ptr(), positions.data_ptr(), active.data_ptr(), out.data_ptr(), batch, tail.shape[0], channels, taps,
+          _dtype(x))
+    return out
+
+
+def scan_dt(low: torch.Tensor, up: torch.Tensor, bias: torch.Tensor) -> torch.Tensor:
+    """fp32 [rows, channels] = softplus(low up^T + bias); low [rows, rank] may be a view."""
+    dev = _dev(up, bias)
+    channels, rank = up.shape
+    _rows_of(low, dev, rank)
+    assert bias.shape == (channels,) and up.dtype == bias.dtype == low.dtype
+    dt = torch.empty(low.shape[0], channels, dtype=torch.float32, device=dev)
+    _call(dev, "nqh_scan_dt", low.data_ptr(), low.stride(0), up.data_ptr(), bias.data_ptr(), dt.data_ptr(), low.shape[0],
+          channels, rank, _dtype(low))
+    return dt
+
+
+def _scan_args(x, dt, bc, z, a_log, skip, state):
+    dev = _dev(x, dt, a_log, skip, state)
+    channels, states = a_log.shape
+    rows = x.shape[0]
+    _rows_of(bc, dev, 2 * states)
+    _rows_of(z, dev, channels)
+    assert x.shape == (rows, channels) and dt.shape == (rows, channels) and dt.dtype == torch.float32
+    assert bc.shape[0] == rows and z.shape[0] == rows and skip.shape == (channels,)
+    assert x.dtype == bc.dtype == z.dtype == a_log.dtype == skip.dtype
+    assert state.dtype == torch.float32 and state.shape[1:] == (states, channels)
+    return dev, rows, channels, states, (x.data_ptr(), dt.data_ptr(), bc.data_ptr(), bc.stride(0), z.data_ptr(), z.stride(0),
+                                         a_log.data_ptr(), skip.data_ptr())
+
+
+def scan_prefill(x: torch.Tensor, dt: torch.Tensor, bc: torch.Tensor, z: torch.Tensor, a_log: torch.Tensor,
+                 skip: torch.Tensor, conv_in: torch.Tensor, state: torch.Tensor, tail: torch.Tensor, layout: PromptPass,
+                 piece_rows: int) -> torch.Tensor:
+    """The pass's tokens through the recurrence: x, dt [rows, channels], bc [rows, B | C], z [rows, channels] (views).  state
+    [slots, states, channels] and tail [slots, taps - 1, channels] (the convolution's last inputs, from conv_in) are moved on
+    IN PLACE at the segments' slots.  Returns (y + skip x) silu(z) [rows, channels]."""
+    dev, rows, channels, states, args = _scan_args(x, dt, bc, z, a_log, skip, state)
+    _dev(state, tail)
+    _rows_of(conv_in, dev, channels)
+    assert rows == layout.rows and conv_in.shape[0] == rows and conv_in.dtype == x.dtype
+    assert tail.dtype == torch.float32 and tail.shape[0] == state.shape[0] and tail.shape[2] == channels
+    assert all(0 <= s[3] < state.shape[0] for s in layout.segments)
+    assert piece_rows >= scan_piece_rows(1, channels, states)
+    pieces, n, chained = layout.pieces(piece_rows)
+    nbytes = _lib.hybrid_lib().nqh_scan_workspace_bytes(n, channels, states) if chained else 0
+    ws = torch.empty(nbytes, dtype=torch.uint8, device=dev) if nbytes else None
+    out = torch.empty(rows, channels, dtype=x.dtype, device=dev)
+    _call(dev, "nqh_scan_prefill", *args, conv_in.data_ptr(), conv_in.stride(0), state.data_ptr(), tail.data_ptr() or None,
+          pieces.data_ptr(), n, int(chained), out.data_ptr(), channels, states, tail.shape[1] + 1, _dtype(x), _ptr(ws), nbytes)
+    return out
+
+
+def scan_step(x: torch.Tensor, dt: torch.Tensor, bc: torch.Tensor, z: torch.Tensor, a_log: torch.Tensor, skip: torch.Tensor,
+              state: torch.Tensor, slots: torch.Tensor, positions: torch.Tensor, active: torch.Tensor) -> torch.Tensor:
+    """The same for one token per sequence, state IN PLACE at the rows' slots.  Idle rows change no state and give zeros."""
+    dev, batch, channels, states, args = _scan_args(x, dt, bc, z, a_log, skip, state)
+    _dev(state, slots, positions, active)
+    assert slots.dtype == torch.int32 and positions.dtype == torch.int64 and active.dtype == torch.bool
+    assert slots.numel() == batch and positions.numel() == batch and active.numel() == batch
+    out = torch.empty(batch, channels, dtype=x.dtype, device=dev)
+    _call(dev, "nqh_scan_step", *args, state.data_ptr(), slots.data_ptr(), positions.data_ptr(), active.data_ptr(),
+          out.data_ptr(), batch, state.shape[0], channels, states, _dtype(x))
     return out
 
 
@@ -263,7 +519,7 @@ def gla_prefill(proj: torch.Tensor, decay: torch.Tensor, state: torch.Tensor, la
     assert all(0 <= s[3] < state.shape[0] for s in layout.segments)
     assert decay.shape == (rows, heads * dim) and decay.dtype == torch.float32
     q, k, v, _, _ = _gla_offsets(proj, heads, dim, vdim, rank)
-    pieces, n, chained = layout.pieces(heads, dim, vdim)
+    pieces, n, chained = layout.pieces(_lib.hybrid_lib().nqh_gla_piece_rows(rows, heads, dim, vdim))
     nbytes = _lib.hybrid_lib().nqh_gla_prefill_workspace_bytes(n, heads, dim, vdim) if chained else 0
     ws = torch.empty(nbytes, dtype=torch.uint8, device=dev) if nbytes else None
     o = torch.empty(rows, heads * vdim, dtype=torch.float32, device=dev)
@@ -361,15 +617,15 @@ def skinny_linear_supported(rows: int, weight: torch.Tensor) -> bool:
 
 
 def skinny_linear(x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor] = None,
-                  out_f32: bool = False) -> torch.Tensor:
-    """x [rows <= 64, in] bf16 @ weight [out, in]^T (+ bias), bf16 or (out_f32) fp32 result."""
+                  out_f32: bool = False, activation: Optional[str] = None, param: float = 0.0) -> torch.Tensor:
+    """activation(x [rows <= 64, in] bf16 @ weight [out, in]^T (+ bias)), bf16 or (out_f32) fp32 result."""
     dev = _dev(x, weight, bias)
     rows, n = x.shape
     assert weight.shape[1] == n and x.dtype == torch.bfloat16 and weight.dtype == torch.bfloat16
     assert bias is None or (bias.shape == (weight.shape[0],) and bias.dtype == torch.bfloat16)
     y = torch.empty(rows, weight.shape[0], dtype=torch.float32 if out_f32 else torch.bfloat16, device=dev)
     _call(dev, "nqh_skinny_linear", x.data_ptr(), weight.data_ptr(), _ptr(bias), y.data_ptr(), rows, weight.shape[0], n,
-          int(out_f32))
+          int(out_f32), ACTIVATIONS[activation], param)
     return y
 
 

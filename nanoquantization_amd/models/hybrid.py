@@ -1,9 +1,10 @@
 """Decoders described layer by layer: specifications and weights.
 
-A DecoderSpec lists layers; each has a mixer (attention over the paged KV cache, or gated linear attention with a
-recurrent state), an optional mixture-of-experts feed-forward, and norms before and after both.  Every constant is a
-field here, so a design is a function from its configuration to a spec plus a table of checkpoint names
-(models/gafulix.py); the engine (engine/hybrid_engine.py) reads the spec only.
+A DecoderSpec lists layers; each has a mixer (attention over the paged KV cache, attention over cached latents, gated linear
+attention or a selective scan with a recurrent state), an optional feed-forward (dense or a mixture of experts), norms before
+and possibly after both, and a residual that is one row per token or several streams.  Every constant is a field here, so a
+design is a function from its configuration to a spec plus a table of checkpoint names (models/gafulix.py,
+models/roletar.py); the engine (engine/hybrid_engine.py) reads the spec only.
 
 Weights are held in the layout the kernels want: projections with a common input side by side in one matrix, the
 experts of a layer stacked.  Checkpoint tensors are copied into views of those (`HybridDecoder.checkpoint_views`)."""
@@ -44,10 +45,36 @@ class AttentionSpec:
     scale: float
     rotary: Optional[RotarySpec] = None
     chunk: int = 0              # > 0: tokens see keys of their own chunk of that many positions only
+    window: int = 0             # > 0: tokens see themselves and the window - 1 tokens before them
+    sink: bool = False          # a learned score per head that takes part in the softmax without key or value
+    bias: bool = True           # of the q, k and v projections
+    qk_norm: bool = True        # RMS norm over the whole q and the whole k projection
 
     def __post_init__(self):
         if self.heads % self.kv_heads:
             raise ValueError(f"{self.heads} query heads do not divide over {self.kv_heads} key/value heads")
+
+
+@dataclass(frozen=True)
+class LatentAttentionSpec:
+    """Keys and values of all heads come from one normalised latent of `rank` elements per token; a rotated key part of
+    rotary.dims elements is shared by all heads.  Query heads are [dim | rotary.dims].  Latent and rotated part are what is
+    cached."""
+    heads: int
+    dim: int
+    vdim: int
+    rank: int
+    scale: float
+    rotary: RotarySpec
+
+
+@dataclass(frozen=True)
+class SelectiveScanSpec:
+    """S = exp(dt A) S + dt x B, y = S C + D x per channel, behind a causal convolution of `taps` tokens."""
+    channels: int
+    state: int
+    dt_rank: int
+    taps: int
 
 
 @dataclass(frozen=True)
@@ -69,17 +96,26 @@ class MoESpec:
 
 
 @dataclass(frozen=True)
+class DenseSpec:
+    """down act(up h); `activation` names one of engine/hybrid_ops.py ACTIVATIONS."""
+    ff: int
+    activation: str
+
+
+@dataclass(frozen=True)
 class LayerSpec:
-    mixer: Union[AttentionSpec, GatedLinearSpec]
-    mlp: Optional[MoESpec]
+    mixer: Union[AttentionSpec, LatentAttentionSpec, GatedLinearSpec, SelectiveScanSpec]
+    mlp: Optional[Union[MoESpec, DenseSpec]]
 
 
 @dataclass(frozen=True)
 class LoopSpec:
-    """Layers start .. stop - 1 run `times` times in a row; passes after the first add the embedding output first."""
+    """Layers start .. stop - 1 run `times` times in a row; passes after the first add the embedding output first if
+    `reinject`."""
     start: int
     stop: int
     times: int
+    reinject: bool = True
 
 
 @dataclass(frozen=True)
@@ -89,11 +125,17 @@ class DecoderSpec:
     eps: float
     layers: Tuple[LayerSpec, ...]
     loop: Optional[LoopSpec] = None
+    post_norms: bool = True           # sublayer outputs are normalised before they are added
+    streams: int = 0                  # > 0: hyper-connections over that many residual streams
+    logit_cap: float = 0.0            # > 0: logits = cap * tanh(logits / cap)
 
     def __post_init__(self):
         lp = self.loop
         if lp is not None and not (0 <= lp.start < lp.stop <= len(self.layers) and lp.times >= 1):
             raise ValueError(f"loop {lp} does not fit {len(self.layers)} layers")
+        if self.streams and (self.post_norms or any(again for _, again in self.runs())
+                             or any(isinstance(l.mlp, MoESpec) for l in self.layers)):
+            raise ValueError("residual streams go with pre-norm layers, dense feed-forwards and loops that add nothing")
 
     def runs(self) -> List[Tuple[int, bool]]:
         """(layer index, whether the embedding output is added in front of it) in execution order.  Every run has its
@@ -103,7 +145,7 @@ class DecoderSpec:
             return [(i, False) for i in range(n)]
         out = [(i, False) for i in range(lp.start)]
         for rep in range(lp.times):
-            out += [(i, rep > 0 and i == lp.start) for i in range(lp.start, lp.stop)]
+            out += [(i, lp.reinject and rep > 0 and i == lp.start) for i in range(lp.start, lp.stop)]
         return out + [(i, False) for i in range(lp.stop, n)]
 
 
@@ -134,9 +176,42 @@ class AttentionWeights(nn.Module):
         super().__init__()
         nq, nk, nv = spec.heads * spec.dim, spec.kv_heads * spec.dim, spec.kv_heads * spec.vdim
         self.splits = (nq, nk, nv)
-        self.qkv, self.qkv_bias = _param(nq + nk + nv, width), _param(nq + nk + nv)
-        self.q_norm, self.k_norm = _param(nq), _param(nk)
+        self.qkv = _param(nq + nk + nv, width)
+        self.qkv_bias = _param(nq + nk + nv) if spec.bias else None
+        self.q_norm, self.k_norm = (_param(nq), _param(nk)) if spec.qk_norm else (None, None)
+        self.sink = _param(spec.heads) if spec.sink else None
         self.out = _param(width, spec.heads * spec.vdim)
+
+
+class LatentAttentionWeights(nn.Module):
+    def __init__(self, spec: LatentAttentionSpec, width: int):
+        super().__init__()
+        rot = spec.rotary.dims
+        self.splits = (spec.heads * (spec.dim + rot), spec.rank + rot)       # queries | latent and rotated key part
+        self.proj = _param(sum(self.splits), width)
+        self.latent_norm = _param(spec.rank)
+        self.expand = _param(spec.heads * (spec.dim + spec.vdim), spec.rank)      # unrotated keys of all heads | values
+        self.out = _param(width, spec.heads * spec.vdim)
+        self.key_rows, self.head_dims = spec.heads * spec.dim, (spec.heads, spec.dim, spec.vdim, spec.rank)
+
+    def per_head(self) -> Tuple[torch.Tensor, torch.Tensor]:
+        """(the key expansion transposed per head [heads, rank, dim], which takes a query into the latent space; the value
+        expansion [heads, vdim, rank])."""
+        H, dim, vdim, rank = self.head_dims
+        keys, values = self.expand.split([H * dim, H * vdim])
+        return keys.view(H, dim, rank).transpose(1, 2).contiguous(), values.view(H, vdim, rank)
+
+
+class SelectiveScanWeights(nn.Module):
+    def __init__(self, spec: SelectiveScanSpec, width: int):
+        super().__init__()
+        C, N, rank = spec.channels, spec.state, spec.dt_rank
+        self.proj = _param(2 * C, width)                                 # x | z
+        self.conv, self.conv_bias = _param(C, spec.taps), _param(C)
+        self.select = _param(rank + 2 * N, C)                            # dt | B | C
+        self.dt_up, self.dt_bias = _param(C, rank), _param(C)
+        self.a_log, self.skip = _param(C, N), _param(C)
+        self.out = _param(width, C)
 
 
 class GatedLinearWeights(nn.Module):
@@ -158,15 +233,43 @@ class MoEWeights(nn.Module):
         self.down = _param(spec.experts, width, spec.ff)
 
 
-class HybridLayer(nn.Module):
-    def __init__(self, spec: LayerSpec, width: int):
+class DenseWeights(nn.Module):
+    def __init__(self, spec: DenseSpec, width: int):
         super().__init__()
-        self.norm_mixer, self.norm_mixer_out = _param(width), _param(width)
-        self.mixer = (AttentionWeights if isinstance(spec.mixer, AttentionSpec) else GatedLinearWeights)(spec.mixer, width)
-        self.mlp = None
+        self.up, self.down = _param(spec.ff, width), _param(width, spec.ff)
+
+
+class StreamWeights(nn.Module):
+    """Hyper-connection of a sublayer: what it reads of every stream, how the old streams [from, to] and its output make the
+    new ones."""
+
+    def __init__(self, streams: int):
+        super().__init__()
+        self.read, self.write, self.mix = _param(streams), _param(streams), _param(streams, streams)
+
+
+WEIGHTS = {AttentionSpec: AttentionWeights, LatentAttentionSpec: LatentAttentionWeights, GatedLinearSpec: GatedLinearWeights,
+           SelectiveScanSpec: SelectiveScanWeights, MoESpec: MoEWeights, DenseSpec: DenseWeights}
+
+
+class HybridLayer(nn.Module):
+    def __init__(self, spec: LayerSpec, width: int, post_norms: bool, streams: int):
+        super().__init__()
+        def norms():
+            return _param(width), _param(width) if post_norms else None
+        self.norm_mixer, self.norm_mixer_out = norms()
+        self.mixer = WEIGHTS[type(spec.mixer)](spec.mixer, width)
+        self.mixer_streams = StreamWeights(streams) if streams else None
+        self.mlp = self.mlp_streams = None
         if spec.mlp is not None:
-            self.norm_mlp, self.norm_mlp_out = _param(width), _param(width)
-            self.mlp = MoEWeights(spec.mlp, width)
+            self.norm_mlp, self.norm_mlp_out = norms()
+            self.mlp = WEIGHTS[type(spec.mlp)](spec.mlp, width)
+            self.mlp_streams = StreamWeights(streams) if streams else None
+
+    def linears(self) -> List[torch.Tensor]:
+        """The matrices of this layer's plain products."""
+        out = [w for n in ("qkv", "proj", "select", "out") if (w := getattr(self.mixer, n, None)) is not None]
+        return out + ([self.mlp.up, self.mlp.down] if isinstance(self.mlp, DenseWeights) else [])
 
 
 class HybridDecoder(nn.Module):
@@ -176,7 +279,7 @@ class HybridDecoder(nn.Module):
         super().__init__()
         self.spec = spec
         self.embed = _param(spec.vocab, spec.width)
-        self.layers = nn.ModuleList([HybridLayer(l, spec.width) for l in spec.layers])
+        self.layers = nn.ModuleList([HybridLayer(l, spec.width, spec.post_norms, spec.streams) for l in spec.layers])
         self.final_norm = _param(spec.width)
         self.head = _param(spec.vocab, spec.width)
 

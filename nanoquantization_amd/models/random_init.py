@@ -51,7 +51,7 @@ def random_awq_qwen3(config: dict, seed: int = 0, std: float = 0.02, device="cud
 
 def random_hybrid(cls, spec, seed: int = 0, device="cuda", dtype=torch.bfloat16):
     """A HybridDecoder subclass with random weights: linears that keep the scale of their input, norms at 1, decays
-    around sigmoid(2)."""
+    around sigmoid(2), scans with step sizes around 0.05 and decay rates 1 .. states, streams that stay apart."""
     with torch.device(device):
         model = cls(spec).to(dtype)
     gen = torch.Generator(device=device).manual_seed(seed)
@@ -60,7 +60,17 @@ def random_hybrid(cls, spec, seed: int = 0, device="cuda", dtype=torch.bfloat16)
             p.data.fill_(1.0)
         elif name.endswith("decay_bias"):
             p.data.fill_(2.0)
-        elif name.endswith("_bias"):
+        elif name.endswith("dt_bias"):
+            p.data.fill_(-3.0)
+        elif name.endswith("a_log"):
+            p.data.copy_(torch.arange(1, p.shape[1] + 1, device=device).log().expand_as(p))
+        elif name.endswith("_streams.read"):
+            p.data.fill_(1.0 / p.numel())
+        elif name.endswith("_streams.mix"):
+            p.data.copy_(0.8 * torch.eye(len(p), device=device) + 0.2 / len(p))
+        elif name.endswith(("skip", "_streams.write")):
+            p.data.fill_(1.0)
+        elif name.endswith(("_bias", "sink")):
             p.data.zero_()
         else:
             flat = p.data.view(p.shape[0], -1)

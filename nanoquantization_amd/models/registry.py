@@ -18,12 +18,21 @@ class Architecture:
     step_kernels: str                                                # the native library its engine needs
 
 
-def _load_gafulix(path: str, cfg: dict, dtype: torch.dtype):
+def _load_hybrid(cls, spec_from_config, path: str, cfg: dict, dtype: torch.dtype):
     from ..utils.loader import load_views, tensor_shapes
-    from .gafulix import GafulixForCausalLM, spec_from_config
-    model = GafulixForCausalLM(spec_from_config(cfg, tensor_shapes(path))).to(dtype)
+    model = cls(spec_from_config(cfg, tensor_shapes(path))).to(dtype)
     load_views(model, path)
     return model
+
+
+def _load_gafulix(path: str, cfg: dict, dtype: torch.dtype):
+    from .gafulix import GafulixForCausalLM, spec_from_config
+    return _load_hybrid(GafulixForCausalLM, spec_from_config, path, cfg, dtype)
+
+
+def _load_roletar(path: str, cfg: dict, dtype: torch.dtype):
+    from .roletar import RoletarForCausalLM, spec_from_config
+    return _load_hybrid(RoletarForCausalLM, spec_from_config, path, cfg, dtype)
 
 
 def _load_qwen3(path: str, cfg: dict, dtype: torch.dtype):
@@ -54,6 +63,7 @@ def _awq_engine():
 
 ARCHITECTURES: List[Architecture] = [
     Architecture("Gafulix", lambda c: c.get("architecture") == "Gafulix", _load_gafulix, _hybrid_engine, "hybrid"),
+    Architecture("Roletar", lambda c: c.get("architecture") == "Roletar", _load_roletar, _hybrid_engine, "hybrid"),
     # Qwen3 with AWQ linears: the reference's checkpoints carry a quantization_config and no further mark
     Architecture("Qwen3Quantized", lambda c: "quantization_config" in c and "architecture" not in c, _load_qwen3,
                  _awq_engine, "awq"),
