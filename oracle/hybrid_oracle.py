@@ -283,3 +283,8 @@ def roletar_logits(config, weights, tokens, dtype=torch.float64, trace=None):
         if trace is not None:
             trace.append(xs.sum(dim=0))
     return softcap(rms(xs.sum(dim=0), w("final.norm"), eps) @ w("head").T, config["logit_softcap"])
+
+
+def logits(config, weights, tokens, dtype=torch.float64, trace=None):
+    """Of the design that the configuration names."""
+    return {"Gafulix": gafulix_logits, "Roletar": roletar_logits}[config["architecture"]](config, weights, tokens, dtype, trace)

@@ -38,7 +38,45 @@ CONFIGS = {
 }
 
 
-def tensor_shapes(cfg, rank=16):
+# Roletar: sliding windows with sinks, latent attention, selective scans, several residual streams
+WIN = dict(type="attention", mixer=dict(heads=6, kv_heads=3, dim=40, vdim=24, scale=0.23, mask=dict(size=17)),
+           mlp=dict(kind="dense", ff=88))
+LATENT = dict(type="latent_attention", mixer=dict(heads=5, dim=24, rot_dim=8, vdim=40, kv_rank=72, scale=0.19,
+                                                  rot=dict(base=700.0, dims=8)), mlp=dict(kind="dense", ff=64))
+SCAN = dict(type="mamba1", mixer=dict(inner=88, state=24, dt_rank=8, conv=4), mlp=None)
+
+
+def latent(mlp="keep", rot_dim=8, base=700.0, **mixer):
+    return layer(LATENT, mlp, rot_dim=rot_dim, rot=dict(base=base, dims=rot_dim), **mixer)
+
+
+def roletar(layers, loop=None, vocab=131, width=72, eps=1e-5, streams=2, cap=12.0):
+    return dict(architecture="Roletar", layers=layers, loop=loop, norm=dict(eps=eps), vocab=vocab, width=width,
+                streams=streams, logit_softcap=cap)
+
+
+# every kind of layer with and without a feed-forward, widths that are and are not multiples of 8, one to eight streams, a
+# window of one, state sizes for one lane and for sixteen per channel, one to seven taps, latents for every kernel form
+CONFIGS.update({
+    "roletar_loop_middle": roletar([layer(SCAN, mlp=WIN["mlp"]), layer(WIN), latent(mlp=None), layer(SCAN, state=16),
+                                    layer(WIN, mlp=None, mask=dict(size=33), heads=4, kv_heads=4), latent(kv_rank=40)],
+                                   dict(start=1, stop=4, times=3), streams=3),
+    "roletar_one_stream": roletar([layer(WIN, mask=dict(size=1), dim=22, vdim=18, heads=4, kv_heads=2),
+                                   layer(SCAN, inner=50, state=5, dt_rank=3, conv=2),
+                                   latent(kv_rank=50, rot_dim=6, dim=22, vdim=26, heads=3)], width=68, vocab=97, streams=1),
+    "roletar_wide": roletar([latent(kv_rank=264, rot_dim=64, dim=128, vdim=96, heads=18, scale=0.07),
+                             layer(SCAN, inner=64, state=130, dt_rank=16, conv=1, mlp=LATENT["mlp"]),
+                             layer(WIN, dim=64, vdim=96, heads=4, kv_heads=1, mask=dict(size=48))],
+                            dict(start=0, stop=3, times=2), width=128, streams=5, cap=3.0),
+    "roletar_many": roletar([layer(SCAN, inner=320, state=33, dt_rank=24, conv=7),
+                             layer(WIN, heads=20, kv_heads=1, dim=16, vdim=32, mask=None),
+                             latent(kv_rank=128, rot_dim=32, dim=32, vdim=160, heads=2)],
+                            dict(start=1, stop=2, times=1), vocab=200, width=80, streams=8, eps=1e-3, cap=40.0),
+    "roletar_no_state": roletar([latent(rot_dim=40, kv_rank=200), layer(WIN, mlp=None)], width=64, streams=4),
+})
+
+
+def _gafulix_shapes(cfg, rank):
     D, shapes = cfg["width"], {"embed": (cfg["vocab"], cfg["width"]), "final.norm": (cfg["width"],),
                                "head": (cfg["vocab"], cfg["width"])}
     for i, l in enumerate(cfg["layers"]):
@@ -66,6 +104,42 @@ def tensor_shapes(cfg, rank=16):
     return shapes
 
 
+def _roletar_shapes(cfg):
+    D, S, shapes = cfg["width"], cfg["streams"], {"embed": (cfg["vocab"], cfg["width"]), "final.norm": (cfg["width"],),
+                                                  "head": (cfg["vocab"], cfg["width"])}
+    for i, l in enumerate(cfg["layers"]):
+        m, p = l["mixer"], f"l{i}."
+        for n in ("1", "2") if l["mlp"] else ("1",):
+            shapes.update({f"{p}norm{n}": (D,), f"{p}hc{n}.in": (S,), f"{p}hc{n}.out": (S,), f"{p}hc{n}.mix": (S, S)})
+        if l["type"] == "attention":
+            H, G = m["heads"], m["kv_heads"]
+            mix = {"q": (H * m["dim"], D), "k": (G * m["dim"], D), "v": (G * m["vdim"], D), "sink": (H,), "o": (D, H * m["vdim"])}
+        elif l["type"] == "latent_attention":
+            H, rank, rot = m["heads"], m["kv_rank"], m["rot_dim"]
+            mix = {"q": (H * (m["dim"] + rot), D), "dkv": (rank + rot, D), "dkv.norm": (rank,), "uk": (H * m["dim"], rank),
+                   "uv": (H * m["vdim"], rank), "o": (D, H * m["vdim"])}
+        else:
+            C, N, rank = m["inner"], m["state"], m["dt_rank"]
+            mix = {"in": (2 * C, D), "conv": (C, m["conv"]), "conv.b": (C,), "x": (rank + 2 * N, C), "dt": (C, rank),
+                   "dt.b": (C,), "A_log": (C, N), "D": (C,), "o": (D, C)}
+        shapes.update({p + "mix." + n: s for n, s in mix.items()})
+        if l["mlp"]:
+            shapes[p + "mlp.up"], shapes[p + "mlp.down"] = (l["mlp"]["ff"], D), (D, l["mlp"]["ff"])
+    return shapes
+
+
+def tensor_shapes(cfg, rank=16):
+    return _roletar_shapes(cfg) if cfg["architecture"] == "Roletar" else _gafulix_shapes(cfg, rank)
+
+
+_per_input = lambda gain: lambda t: t * gain * t.shape[-1] ** -0.5
+# squared activations and repeated passes amplify rounding: gains low enough that bf16 is not chaotic
+_ROLETAR_INIT = {"sink": lambda t: 2.0 + t, "A_log": lambda t: torch.arange(1.0, t.shape[1] + 1).log() - 2.0 + 0.5 * t,
+                 "D": lambda t: 1.0 + 0.5 * t, "in": lambda t: _per_input(1.0)(t) if t.dim() == 2 else 0.5 + 0.2 * t,
+                 "out": lambda t: 0.6 + 0.3 * t, "mix": lambda t: torch.eye(len(t)) + 0.1 * t, "up": _per_input(1.0),
+                 "down": _per_input(0.4), "uk": _per_input(1.0), "o": _per_input(1.0)}
+
+
 def random_weights(cfg, seed=0, rank=16, clear_routing=False):
     """bf16 weights: linears that keep their input's scale, norm weights around 1, biases and decays that matter.
     `clear_routing`: the first 8 dimensions hold the token's class, no sublayer writes them and the routers read nothing
@@ -77,6 +151,10 @@ def random_weights(cfg, seed=0, rank=16, clear_routing=False):
         last = name.split(".")[-1]
         if "norm" in last:
             t = 1.0 + 0.3 * t
+        elif cfg["architecture"] == "Roletar" and last in _ROLETAR_INIT:
+            t = _ROLETAR_INIT[last](t)
+        elif name.endswith("dt.b"):
+            t = t - 1.5                             # memories of a few tokens and of hundreds
         elif last == "b":
             t = t + 2.0 if ".a2." in name else 0.3 * t
         elif name == "embed":

@@ -38,7 +38,7 @@ _oracle = {}
 def expected(name, weights, ids):
     key = (name, id(weights), tuple(ids))
     if key not in _oracle:
-        _oracle[key] = o.gafulix_logits(CONFIGS[name], weights, ids)
+        _oracle[key] = o.logits(CONFIGS[name], weights, ids)
     return _oracle[key]
 
 
@@ -62,6 +62,10 @@ def run(eng, ids, cuts, lease=None):
     return torch.cat(out)
 
 
+def free_of(eng):
+    return sorted(eng.cache.free), sorted(eng.states.free) if eng.states is not None else None
+
+
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("name", sorted(CONFIGS))
 def test_prompt_portions_and_decoding_against_oracle(models, name, dtype):
@@ -70,12 +74,28 @@ def test_prompt_portions_and_decoding_against_oracle(models, name, dtype):
     ids = tokens(T, V, seed=3)
     want = expected(name, w, ids)
     eng = HybridEngine(model, max_batch=1, max_seq_len=128, block_size=16)
-    free = (len(eng.cache.free), len(eng.states.free))
+    free = free_of(eng)
     for cuts in ([T], [1], [40], [2] * 36, [3, 2, 16, 1, 7, 2, 30], [19, 1, 1, 20, 2]):
         print(f"{name} {dtype} cuts {cuts[:4]}", flush=True)
         got = run(eng, ids, cuts)
         assert logit_error(got, want) <= TOL[dtype], (name, dtype, cuts[:4], logit_error(got, want))
-    assert (len(eng.cache.free), len(eng.states.free)) == free
+    assert free_of(eng) == free
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("name", [n for n in sorted(CONFIGS) if n.startswith("roletar")])
+def test_latent_passes_of_every_form_agree(models, name, dtype):
+    """The same portions with their latents expanded, and absorbed into the queries: all of the prompt in one pass, and the
+    second half after the first."""
+    model, _, w = models(name, dtype)
+    ids = tokens(71, CONFIGS[name]["vocab"], seed=3)
+    want = expected(name, w, ids)
+    for limit in (0, 10 ** 6):
+        eng = HybridEngine(model, max_batch=1, max_seq_len=128, block_size=16)
+        eng.absorb_rows = limit
+        for cuts in ([71], [30, 2, 39]):
+            print(f"{name} {dtype} absorbing up to {limit} rows, cuts {cuts}", flush=True)
+            assert logit_error(run(eng, ids, cuts), want) <= TOL[dtype], (name, dtype, limit, cuts)
 
 
 def test_residual_stream_after_every_layer(models):
@@ -87,15 +107,15 @@ def test_residual_stream_after_every_layer(models):
         print(f"{name} layer trace", flush=True)
         a = eng.extend([Portion(lease, 0, ids, [22])], trace=got).clone()
         assert torch.allclose(a, eng.extend([Portion(lease, 0, ids, [22])]), atol=1e-5)     # tracing changes nothing
-        o.gafulix_logits(CONFIGS[name], w, ids, trace=want)
+        o.logits(CONFIGS[name], w, ids, trace=want)
         assert len(got) == len(want) == len(eng.runs)
         for g, e in zip(got, want):
             assert (g.double().cpu() - e).abs().max() <= 2e-5 * e.abs().max()
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-def test_unequal_requests_in_one_batch_equal_each_alone(models, dtype):
-    name = "loop_middle"
+@pytest.mark.parametrize("name", ["loop_middle", "roletar_loop_middle", "roletar_wide"])
+def test_unequal_requests_in_one_batch_equal_each_alone(models, name, dtype):
     model, _, w = models(name, dtype)
     V = CONFIGS[name]["vocab"]
     lens, steps = [1, 45, 20, 33, 2], 6
@@ -124,9 +144,9 @@ def test_unequal_requests_in_one_batch_equal_each_alone(models, dtype):
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-def test_blocks_and_slots_used_again(models, dtype):
+@pytest.mark.parametrize("name", ["no_loop", "roletar_one_stream", "roletar_many"])
+def test_blocks_and_slots_used_again(models, name, dtype):
     """One sequence's worth of blocks and one slot, handed from request to request in a different order every time."""
-    name = "no_loop"
     model, _, w = models(name, dtype)
     V = CONFIGS[name]["vocab"]
     eng = HybridEngine(model, max_batch=1, max_seq_len=64, block_size=16, num_blocks=4, num_slots=1)
@@ -141,9 +161,9 @@ def test_blocks_and_slots_used_again(models, dtype):
     eng.release(a)
 
 
-def test_long_decoding_stays_on_the_oracle(models):
-    """Every chunk edge, block border and wrap is passed by single decoded tokens."""
-    name = "loop_all"
+@pytest.mark.parametrize("name", ["loop_all", "roletar_loop_middle"])
+def test_long_decoding_stays_on_the_oracle(models, name):
+    """Every chunk edge, window, block border and wrap is passed by single decoded tokens."""
     for dtype in (torch.float32, torch.bfloat16):
         model, _, w = models(name, dtype)
         ids = tokens(150, CONFIGS[name]["vocab"], seed=8)
@@ -152,8 +172,8 @@ def test_long_decoding_stays_on_the_oracle(models):
         assert logit_error(run(eng, ids, [1]), expected(name, w, ids)) <= TOL[dtype]
 
 
-def test_graph_replays_equal_eager_steps(models):
-    name = "loop_middle"
+@pytest.mark.parametrize("name", ["loop_middle", "roletar_loop_middle"])
+def test_graph_replays_equal_eager_steps(models, name):
     model, _, _ = models(name, torch.bfloat16)
     ids = tokens(40, CONFIGS[name]["vocab"], seed=9)
     outs = []
@@ -174,11 +194,11 @@ def test_graph_replays_equal_eager_steps(models):
     assert torch.equal(outs[0], outs[1])
 
 
+@pytest.mark.parametrize("name", ["loop_all", "roletar_loop_middle"])
 @pytest.mark.parametrize("rows", [20, 40, 70])
-def test_wider_batches_with_and_without_graph(models, rows):
+def test_wider_batches_with_and_without_graph(models, rows, name):
     """Enough rows for the other forms of the linears and experts (and, at 70, for the library's products, which stay out
     of a graph): the same tokens from graph replays and from eager steps, for unequal requests that come and go."""
-    name = "loop_all"
     model, _, _ = models(name, torch.bfloat16)
     V = CONFIGS[name]["vocab"]
     reqs = [(tokens(1 + (7 * i) % 23, V, seed=200 + i), 3 + i % 9) for i in range(rows + 7)]
@@ -195,16 +215,17 @@ def test_wider_batches_with_and_without_graph(models, rows):
 def greedy_reference(name, weights, prompt, new):
     seq, gaps = list(prompt), []
     for _ in range(new):
-        top = o.gafulix_logits(CONFIGS[name], weights, seq)[-1].topk(2)
+        top = o.logits(CONFIGS[name], weights, seq)[-1].topk(2)
         gaps.append((top.values[0] - top.values[1]).item())
         seq.append(top.indices[0].item())
     return seq[len(prompt):], gaps
 
 
-def test_generate_and_serve_greedy(models):
+@pytest.mark.parametrize("name", ["one_pass_loop", "roletar_loop_middle"])
+def test_generate_and_serve_greedy(models, name):
     """Through the schedulers: the fp32 engine picks the oracle's tokens; requests of any lengths, rows, blocks and slots
     recycled, long prompts in portions."""
-    name, new = "one_pass_loop", 8
+    new = 8
     model, _, w = models(name, torch.float32)
     V = CONFIGS[name]["vocab"]
     prompts = [tokens(n, V, seed=70 + n) for n in (19, 19, 19)]
@@ -238,8 +259,9 @@ def test_generate_and_serve_greedy(models):
     assert all(eos not in c[:-1] for c in cut)
 
 
-def test_command_line_generates(models, tmp_path):
-    _, path, _ = models("no_loop", torch.bfloat16)
+@pytest.mark.parametrize("name", ["no_loop", "roletar_one_stream"])
+def test_command_line_generates(models, tmp_path, name):
+    _, path, _ = models(name, torch.bfloat16)
     cmd = [sys.executable, "-m", "nanoquantization_amd.generate", "--model", str(path), "--max-new-tokens", "5",
            "--prompt-ids", "3,1,4", "--prompt-ids", "15,9,2,6"]
     print("cli", flush=True)
@@ -250,8 +272,8 @@ def test_command_line_generates(models, tmp_path):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-def test_trace_runner(models, tmp_path, dtype):
-    name = "loop_middle"
+@pytest.mark.parametrize("name", ["loop_middle", "roletar_loop_middle"])
+def test_trace_runner(models, tmp_path, name, dtype):
     _, path, w = models(name, torch.bfloat16)
     V = CONFIGS[name]["vocab"]
     a, b = tokens(40, V, seed=21), tokens(9, V, seed=22)

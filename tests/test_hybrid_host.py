@@ -8,12 +8,14 @@ import re
 import pytest
 import torch
 
-from hybrid_cases import ATT, CONFIGS, GLA, config, layer, random_weights, tensor_shapes, tokens, write_checkpoint
+from hybrid_cases import (ATT, CONFIGS, GLA, LATENT, WIN, config, latent, layer, random_weights, roletar, tensor_shapes, tokens,
+                          write_checkpoint)
 from nanoquantization_amd import _lib
 from nanoquantization_amd.engine.cache import PagedKVCache, RecurrentStateCache
 from nanoquantization_amd.models import registry
 from nanoquantization_amd.models.gafulix import GafulixForCausalLM, spec_from_config
-from nanoquantization_amd.models.hybrid import RotarySpec, YarnScaling, rotary_table
+from nanoquantization_amd.models.hybrid import DecoderSpec, RotarySpec, YarnScaling, rotary_table
+from nanoquantization_amd.models.roletar import spec_from_config as roletar_spec
 from nanoquantization_amd.utils.loader import model_from_config, save_views
 from oracle import hybrid_oracle as o
 
@@ -47,7 +49,7 @@ def test_checkpoint_round_trip_and_views(name, tmp_path):
     cfg, w = CONFIGS[name], random_weights(CONFIGS[name], rank=12)
     write_checkpoint(tmp_path, cfg, w)
     m = model_from_config(str(tmp_path))
-    assert isinstance(m, GafulixForCausalLM)
+    assert type(m).__name__ == cfg["architecture"] + "ForCausalLM"
     views = m.checkpoint_views()
     assert {k: tuple(v.shape) for k, v in views.items()} == {k: tuple(s) for k, s in tensor_shapes(cfg, 12).items()}
     for k, v in views.items():
@@ -76,7 +78,45 @@ def test_loader_rejects_what_does_not_fit(tmp_path):
     model_from_config(str(tmp_path))
 
 
+def test_roletar_configuration(tmp_path):
+    cfg = CONFIGS["roletar_loop_middle"]
+    spec = roletar_spec(cfg)
+    assert spec.runs() == [(i, False) for i in (0, 1, 2, 3, 1, 2, 3, 1, 2, 3, 4, 5)] and o.layer_schedule(cfg)[4] == (1, True)
+    assert (spec.streams, spec.logit_cap, spec.post_norms) == (3, 12.0, False)
+    a, l, s = spec.layers[1].mixer, spec.layers[2].mixer, spec.layers[0].mixer
+    assert (a.window, a.chunk, a.sink, a.bias, a.qk_norm, a.rotary) == (17, 0, True, False, False, None)
+    assert (l.rank, l.rotary) == (72, RotarySpec(8, 700.0)) and (s.channels, s.state, s.dt_rank, s.taps) == (88, 24, 8, 4)
+    assert spec.layers[2].mlp is None and spec.layers[0].mlp.activation == "relu2"
+    assert roletar_spec(CONFIGS["roletar_many"]).layers[1].mixer.window == 0
+    for bad in (layer(WIN, kv_heads=4), layer(LATENT, rot=dict(base=10.0, dims=4)), dict(WIN, type="gla"),
+                dict(WIN, mlp=dict(kind="moe", ff=8))):
+        with pytest.raises(ValueError):
+            roletar_spec(roletar([bad]))
+    with pytest.raises(ValueError):          # what streams do not go with
+        DecoderSpec(vocab=8, width=8, eps=0.1, layers=(), streams=2)
+    w = random_weights(cfg)
+    w["l3.norm2"], w["l3.hc2.in"] = torch.ones(72), torch.ones(3)      # of a feed-forward that layer 3 does not have
+    write_checkpoint(tmp_path, cfg, w)
+    m = model_from_config(str(tmp_path), dtype=torch.float32)
+    into, out_of = m.layers[2].mixer.per_head()
+    uk, uv = w["l2.mix.uk"].float(), w["l2.mix.uv"].float()
+    assert torch.equal(into[3], uk[3 * 24:4 * 24].T) and torch.equal(out_of[4], uv[4 * 40:])
+    assert len(m.layers[0].linears()) == 5 and len(m.layers[2].linears()) == 2
+    del w["l1.mix.sink"]
+    write_checkpoint(tmp_path, cfg, w)
+    with pytest.raises(ValueError):
+        model_from_config(str(tmp_path))
+
+
+def test_cache_rows_of_latents():
+    from nanoquantization_amd.engine.hybrid_ops import latent_row
+    bf, fp = torch.bfloat16, torch.float32
+    assert latent_row(512, 64, bf) == (512, 576) and latent_row(50, 6, bf) == (64, 96) and latent_row(65, 33, bf) == (128, 192)
+    assert latent_row(50, 6, fp) == (50, 56) and latent_row(600, 64, bf) == (600, 664) and latent_row(64, 80, bf) == (64, 144)
+
+
 def test_registry_picks_by_config(tmp_path):
+    assert registry.find_architecture({"architecture": "Roletar"}).step_kernels == "hybrid"
     assert registry.find_architecture({"architecture": "Gafulix"}).name == "Gafulix"
     assert registry.find_architecture({"quantization_config": {}}).name == "Qwen3Quantized"
     with pytest.raises(ValueError):
@@ -129,6 +169,8 @@ def test_caches_hand_out_and_take_back():
     assert sorted(c.free) == list(range(5))
     s = RecurrentStateCache(2, [None, (3, 4, 5)], "cpu")
     assert s.state[0] is None and s.state[1].shape == (2, 3, 4, 5) and s.state[1].dtype == torch.float32
+    t = RecurrentStateCache(3, [(2, 6), None], "cpu", [(4, 6), None])
+    assert t.tail[0].shape == (3, 4, 6) and t.tail[1] is None and s.tail == [None, None]
     x, y = s.allocate(), s.allocate()
     assert {x, y} == {0, 1}
     with pytest.raises(RuntimeError):
@@ -152,6 +194,45 @@ def test_oracle_mechanisms_consistent():
     whole = o.attend(q, k, v, 0.7, chunk=4)
     parts = torch.cat([o.attend(q[i:i + 4], k[i:i + 4], v[i:i + 4], 0.7) for i in range(0, 9, 4)])
     assert torch.allclose(whole, parts)
+    # a window as a matrix, a sink as a further key that scores it and has no value
+    s = torch.einsum("ihd,jhd->hij", q, k) * 0.7
+    i, j = torch.arange(9).view(9, 1), torch.arange(9)
+    s = s.masked_fill(~((j <= i) & (i - j < 4)), -torch.inf)
+    sink = torch.tensor([0.3, 5.0]).double()
+    p = torch.softmax(torch.cat([s, sink.view(2, 1, 1).expand(2, 9, 1)], -1), -1)[..., :9]
+    assert torch.allclose(o.attend(q, k, v, 0.7, window=4, sink=sink), torch.einsum("hij,jhd->ihd", p, v))
+    # latent attention as plain attention over expanded keys that repeat the shared part
+    wl = {n: torch.randn(*sh, generator=g).double() for n, sh in dict(q=(2 * 7, 6), dkv=(5 + 4, 6), uk=(2 * 3, 5), uv=(2 * 4, 5),
+                                                                      o=(6, 8)).items()}
+    wl["dkv.norm"] = torch.rand(5, generator=g).double()
+    h = torch.randn(4, 6, generator=g).double()
+    got = o.latent_attention_mixer(h, wl, dict(heads=2, dim=3, rot_dim=4, vdim=4, kv_rank=5, scale=0.4, rot=dict(base=9.0)), 1e-3)
+    down = h @ wl["dkv"].T
+    c = o.rms(down[:, :5], wl["dkv.norm"], 1e-3)
+    z = torch.polar(torch.ones(4, 2).double(), torch.arange(4).view(4, 1) * torch.tensor([1.0, 1 / 3]).double())
+    turn = lambda x: torch.view_as_real(torch.view_as_complex(x.reshape(4, -1, 2, 2).contiguous()) * z.unsqueeze(1)).reshape(4, -1, 4)
+    qq = (h @ wl["q"].T).view(4, 2, 7)
+    kk = torch.cat([(c @ wl["uk"].T).view(4, 2, 3), turn(down[:, 5:]).expand(4, 2, 4)], -1)
+    s = torch.einsum("ihd,jhd->hij", torch.cat([qq[..., :3], turn(qq[..., 3:])], -1), kk) * 0.4
+    p = torch.softmax(s.masked_fill(j[:4] > i[:4], -torch.inf), -1)
+    assert torch.allclose(got, torch.einsum("hij,jhd->ihd", p, (c @ wl["uv"].T).view(4, 2, 4)).reshape(4, 8) @ wl["o"].T)
+    # the scan written out as a sum, and cut in two
+    x, dt, A = torch.randn(6, 3, generator=g).double(), torch.rand(6, 3, generator=g).double(), -torch.rand(3, 4, generator=g).double()
+    B, C, D = torch.randn(6, 4, generator=g).double(), torch.randn(6, 4, generator=g).double(), torch.randn(3, generator=g).double()
+    y, S = o.selective_scan(x, dt, A, B, C, D)
+    want = sum((torch.exp(dt[u + 1:6].sum(0)[:, None] * A) * (dt[u] * x[u])[:, None] * B[u]) @ C[5] for u in range(6)) + D * x[5]
+    assert torch.allclose(y[5], want)
+    y1, S1 = o.selective_scan(x[:2], dt[:2], A, B[:2], C[:2], D)
+    y2, S2 = o.selective_scan(x[2:], dt[2:], A, B[2:], C[2:], D, S1)
+    assert torch.allclose(torch.cat([y1, y2]), y) and torch.allclose(S2, S)
+    wc, bc = torch.randn(3, 4, generator=g).double(), torch.randn(3, generator=g).double()
+    conv = o.short_conv(x, wc, bc)
+    assert torch.allclose(conv[1], wc[:, 3] * x[1] + wc[:, 2] * x[0] + bc)
+    assert torch.allclose(o.short_conv(x[3:], wc, bc, x[:3]), conv[3:])
+    # hyper-connections that only add are the plain residual
+    xs = torch.stack([x, x * 0])
+    new = o.hyper_write(xs, torch.tensor([[1.0, 0.5], [0.0, 1.0]]).double(), torch.tensor([1.0, 0.0]).double(), dt)
+    assert torch.allclose(new[0], x + dt) and torch.allclose(new[1], 0.5 * x)
     cfg = CONFIGS["one_pass_loop"]
     w = random_weights(cfg)
     ids = tokens(6, cfg["vocab"])
