@@ -183,8 +183,9 @@ def gemv_kernel_name(M, N, K, dtype_name, g=G):
     return f"{kern} (plan {name}, split {sp.value})"
 
 
-# Sizes of the --hybrid option: the layers of Qwen3-0.6B and Qwen3-8B, and a Gafulix model whose attention layers have the
-# same heads and whose experts that a token uses add up to the same feed-forward width.
+# Sizes of the --hybrid option: the layers of Qwen3-0.6B and Qwen3-8B, a Gafulix model whose attention layers have the
+# same heads and whose experts that a token uses add up to the same feed-forward width, and a Roletar model whose
+# feed-forwards (two matrices instead of three) take the same number of operations.
 HYBRID_SIZES = {
     "0.6b_layers": dict(width=1024, heads=16, kv_heads=8, inter=3072, layers=6),
     "8b_layers": dict(width=4096, heads=32, kv_heads=8, inter=12288, layers=6),
@@ -205,27 +206,52 @@ def gafulix_bench_config(size, chunk=8192, experts=8, top=2):
             "norm": {"eps": 1e-6}, "vocab": HYBRID_VOCAB, "width": s["width"]}
 
 
-def hybrid_models(size, dev):
-    """The two models of a size: (name, model, engine class)."""
+def roletar_bench_config(size, window=8192, streams=2):
+    """Layers attention, selective scan, latent attention, ...; windows longer than the bench's contexts."""
+    s = HYBRID_SIZES[size]
+    mlp = {"kind": "dense", "ff": 3 * s["inter"] // 2}
+    mixers = {"attention": {"heads": s["heads"], "kv_heads": s["kv_heads"], "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                            "mask": {"size": window}},
+              "mamba1": {"inner": 2 * s["width"], "state": 16, "dt_rank": s["width"] // 16, "conv": 4},
+              "latent_attention": {"heads": s["heads"], "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512,
+                                   "scale": 192 ** -0.5, "rot": {"base": 10000.0, "dims": 64}}}
+    kinds = list(mixers)
+    return {"architecture": "Roletar", "loop": None, "norm": {"eps": 1e-6}, "vocab": HYBRID_VOCAB, "width": s["width"],
+            "streams": streams, "logit_softcap": 30.0,
+            "layers": [{"type": kinds[i % 3], "mixer": mixers[kinds[i % 3]], "mlp": mlp} for i in range(s["layers"])]}
+
+
+HYBRID_MODELS = ("gafulix", "roletar", "qwen3_awq")
+
+
+def hybrid_models(size, dev, names=HYBRID_MODELS):
+    """The models of a size: (name, model, engine class)."""
     from nanoquantization_amd.engine import HybridEngine, LLMEngine
-    from nanoquantization_amd.models.gafulix import GafulixForCausalLM, spec_from_config
+    from nanoquantization_amd.models import gafulix, roletar
     from nanoquantization_amd.models.random_init import QWEN3_0P6B, random_awq_qwen3, random_hybrid
     s = HYBRID_SIZES[size]
-    yield "gafulix", random_hybrid(GafulixForCausalLM, spec_from_config(gafulix_bench_config(size)), device=dev), HybridEngine
+    if "gafulix" in names:
+        spec = gafulix.spec_from_config(gafulix_bench_config(size))
+        yield "gafulix", random_hybrid(gafulix.GafulixForCausalLM, spec, device=dev), HybridEngine
+    if "roletar" in names:
+        spec = roletar.spec_from_config(roletar_bench_config(size))
+        yield "roletar", random_hybrid(roletar.RoletarForCausalLM, spec, device=dev), HybridEngine
+    if "qwen3_awq" not in names:
+        return
     qwen = dict(QWEN3_0P6B, num_hidden_layers=s["layers"], vocab_size=HYBRID_VOCAB, hidden_size=s["width"],
                 total_num_heads=s["heads"], total_num_kv_heads=s["kv_heads"], intermediate_size=s["inter"],
                 max_position_embeddings=16384, tie_word_embeddings=False)
     yield "qwen3_awq", random_awq_qwen3(qwen, device=dev), LLMEngine
 
 
-def hybrid_bench(sizes, new=48):
-    """Prefill and decode throughput of Gafulix models beside AWQ Qwen3 models of the same layer sizes."""
+def hybrid_bench(sizes, names=HYBRID_MODELS, new=48):
+    """Prefill and decode throughput of the hybrid decoders and of AWQ Qwen3 models of the same layer sizes."""
     dev = torch.device("cuda:0")
-    out = {"metric": "prefill and decode tok/s, Gafulix (bf16) beside Qwen3 (AWQ W4A16) at equal layer sizes", "n_gpus": 1,
+    out = {"metric": "prefill and decode tok/s, Gafulix and Roletar (bf16) beside Qwen3 (AWQ W4A16) at equal layer sizes", "n_gpus": 1,
            "data": "synthetic", "dtype": "bf16", "higher_is_better": True, "sizes": {}}
     for size in sizes:
         res = out["sizes"][size] = {"config": dict(HYBRID_SIZES[size], vocab=HYBRID_VOCAB)}
-        for name, model, engine in hybrid_models(size, dev):
+        for name, model, engine in hybrid_models(size, dev, names):
             r = res[name] = {}
             for batch, plen in ((1, 512), (1, 2048), (1, 8192), (16, 2048), (64, 512)):
                 eng = engine(model, max_batch=batch, max_seq_len=plen + new, block_size=64)
@@ -245,17 +271,20 @@ def hybrid_bench(sizes, new=48):
                 torch.cuda.empty_cache()
             del model
             torch.cuda.empty_cache()
-        for case, g in res["gafulix"].items():
-            q = res["qwen3_awq"][case]
-            g["prefill_vs_qwen3"] = round(g["prefill_tok_per_s"] / q["prefill_tok_per_s"], 3)
-            g["decode_vs_qwen3"] = round(g["decode_tok_per_s"] / q["decode_tok_per_s"], 3)
+        for name, other, label in (("gafulix", "qwen3_awq", "qwen3"), ("roletar", "gafulix", "gafulix"),
+                                   ("roletar", "qwen3_awq", "qwen3")):
+            for case, g in res.get(name, {}).items():
+                q = res.get(other, {}).get(case)
+                if q:
+                    g[f"prefill_vs_{label}"] = round(g["prefill_tok_per_s"] / q["prefill_tok_per_s"], 3)
+                    g[f"decode_vs_{label}"] = round(g["decode_tok_per_s"] / q["decode_tok_per_s"], 3)
     return out
 
 
 def hybrid_one(size, which, batch, plen, new):
     """One prefill and `new` decode steps of one model, nothing timed: the subject of a rocprofv3 run (the steps run
     without a graph, so that every launch has its name)."""
-    for name, model, engine in hybrid_models(size, torch.device("cuda:0")):
+    for name, model, engine in hybrid_models(size, torch.device("cuda:0"), (which,)):
         if name == which:
             eng = engine(model, max_batch=batch, max_seq_len=plen + new, block_size=64, use_graph=False)
             ids = torch.randint(0, HYBRID_VOCAB, (batch, plen), generator=torch.Generator().manual_seed(1)).tolist()
@@ -267,10 +296,11 @@ def hybrid_one(size, which, batch, plen, new):
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--hybrid", action="store_true",
-                    help="instead of the default workload: Gafulix beside AWQ Qwen3 at equal layer sizes, one JSON line")
+                    help="instead of the default workload: Gafulix, Roletar and AWQ Qwen3 at equal layer sizes, one JSON line")
     ap.add_argument("--hybrid-size", choices=sorted(HYBRID_SIZES), action="append", help="with --hybrid: only this size")
+    ap.add_argument("--hybrid-model", choices=HYBRID_MODELS, action="append", help="with --hybrid: only this model")
     ap.add_argument("--hybrid-one", nargs=4, metavar=("MODEL", "BATCH", "PROMPT", "NEW"),
-                    help="with --hybrid: one run of gafulix|qwen3_awq for a profiler, nothing timed")
+                    help="with --hybrid: one run of gafulix|roletar|qwen3_awq for a profiler, nothing timed")
     ap.add_argument("--one", nargs=4, metavar=("KIND", "K", "N", "M"),
                     help="launch one problem a few times for a profiler: linear|dequant|copy K N M")
     ap.add_argument("--one-dtype", choices=["bf16", "f16"], default="bf16")
@@ -309,7 +339,7 @@ def main():
         if args.hybrid_one:
             hybrid_one(sizes[0], args.hybrid_one[0], *map(int, args.hybrid_one[1:]))
         else:
-            print(json.dumps(hybrid_bench(sizes)))
+            print(json.dumps(hybrid_bench(sizes, args.hybrid_model or HYBRID_MODELS)))
         return
     if args.one:
         kind, K1, N1, M1 = args.one[0], int(args.one[1]), int(args.one[2]), int(args.one[3])

@@ -400,7 +400,8 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
 
 // Decode attention.  Workgroup = (sequence, kv head, 16 of its query heads, context split); a wave takes tiles of 32 keys
 // through its own part of LDS, no barriers until the merge.  RL > 0: latent attention, the first RL elements of a key row are
-// the value row.
+// the value row; they and the rest lie in two tiles whose row widths are powers of two, so that a load-to-LDS takes whole
+// rows and needs next to no address arithmetic.
 template <int R, int WAVES, int RL>
 __global__ __launch_bounds__(64 * WAVES) void attn_decode_kernel(
     const uint16_t* __restrict__ q, const uint16_t* __restrict__ k_cache, const uint16_t* __restrict__ v_cache,
@@ -408,7 +409,9 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_kernel(
     uint16_t* __restrict__ out, float* __restrict__ partial, int heads, int kv_heads, int vdim, int block_size, int max_blocks,
     int num_blocks, int chunk, int window, float scale, int splits, int head_tiles) {
     using L = RowLayout<R>;
-    constexpr int RV = RL > 0 ? RL : R, RS = RV + 2;      // value elements, width of a result row
+    using LL = RowLayout<RL == 0 ? 32 : RL>;
+    using LR = RowLayout<RL == 0 ? 32 : R - RL>;
+    constexpr int RV = RL > 0 ? RL : R, RS = RV + 4;      // value elements, width of a result row
     constexpr int TT = 32, kBytes = TT * R * 2, kLoads = kBytes / 1024;
     constexpr int kWave = RL > 0 ? kBytes : 2 * kBytes + 1024;
     static_assert(RV <= R && 16 * RS * 4 <= kWave && WAVES * kWave <= 160 * 1024, "the per-wave results reuse the wave's tiles");
@@ -448,14 +451,14 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_kernel(
         int blk = table[j / block_size];
         blk = blk < 0 ? 0 : (blk >= num_blocks ? num_blocks - 1 : blk);
         const int my_row = (blk * kv_heads + g) * block_size + j % block_size;
-#pragma unroll
-        for (int i = 0; i < kLoads; ++i) {
-            const int n = i * 64 + lane, row = n / L::kPieces;
-            const int64_t base = (int64_t)__shfl(my_row, row) * R;
-            __builtin_amdgcn_global_load_lds(NQH_GPTR(k_cache + base + L::k_source(row, n % L::kPieces)),
-                                             NQH_LPTR(kt + i * 1024), 16, 0, 0);
-        }
         if constexpr (RL == 0) {
+#pragma unroll
+            for (int i = 0; i < kLoads; ++i) {
+                const int n = i * 64 + lane, row = n / L::kPieces;
+                const int64_t base = (int64_t)__shfl(my_row, row) * R;
+                __builtin_amdgcn_global_load_lds(NQH_GPTR(k_cache + base + L::k_source(row, n % L::kPieces)),
+                                                 NQH_LPTR(kt + i * 1024), 16, 0, 0);
+            }
 #pragma unroll
             for (int i = 0; i < kLoads; ++i) {
                 const int n = i * 64 + lane, row = n / L::kPieces;
@@ -466,15 +469,40 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_kernel(
             // a wave's loads return in order: with at most the V tile's outstanding, the K tile has landed
             asm volatile("s_waitcnt vmcnt(%0)" : : "n"(kLoads) : "memory");
         } else {
+#pragma unroll
+            for (int i = 0; i < LL::kPieces / 2; ++i) {
+                const int n = i * 64 + lane, row = n / LL::kPieces;
+                const int64_t base = (int64_t)(LL::kPieces == 64 ? __builtin_amdgcn_readlane(my_row, i) : __shfl(my_row, row)) * R;
+                __builtin_amdgcn_global_load_lds(NQH_GPTR(k_cache + base + LL::k_source(row, n % LL::kPieces)),
+                                                 NQH_LPTR(kt + i * 1024), 16, 0, 0);
+            }
+#pragma unroll
+            for (int i = 0; i < LR::kPieces / 2; ++i) {
+                const int n = i * 64 + lane, row = n / LR::kPieces;
+                const int64_t base = (int64_t)__shfl(my_row, row) * R + RL;
+                __builtin_amdgcn_global_load_lds(NQH_GPTR(k_cache + base + LR::k_source(row, n % LR::kPieces)),
+                                                 NQH_LPTR(kt + TT * RL * 2 + i * 1024), 16, 0, 0);
+            }
             asm volatile("s_waitcnt vmcnt(0)" : : : "memory");
         }
         f32x4 st[2];
+        st[0] = st[1] = f32x4{0.f, 0.f, 0.f, 0.f};
+        if constexpr (RL == 0) {
 #pragma unroll
-        for (int a = 0; a < 2; ++a) {
-            st[a] = f32x4{0.f, 0.f, 0.f, 0.f};
+            for (int a = 0; a < 2; ++a)
+#pragma unroll
+                for (int s = 0; s < R / 32; ++s)
+                    st[a] = Bf::mfma16(*reinterpret_cast<const u32x4*>(kt + L::k_at(16 * a + lo, 4 * s + hi)), bq[s], st[a]);
+        } else {
 #pragma unroll
             for (int s = 0; s < R / 32; ++s)
-                st[a] = Bf::mfma16(*reinterpret_cast<const u32x4*>(kt + L::k_at(16 * a + lo, 4 * s + hi)), bq[s], st[a]);
+#pragma unroll
+                for (int a = 0; a < 2; ++a) {
+                    const int row = 16 * a + lo;
+                    const unsigned char* p = s < RL / 32 ? kt + LL::k_at(row, 4 * s + hi)
+                                                         : kt + TT * RL * 2 + LR::k_at(row, 4 * (s - RL / 32) + hi);
+                    st[a] = Bf::mfma16(*reinterpret_cast<const u32x4*>(p), bq[s], st[a]);
+                }
         }
         float mx = kNegBig;
 #pragma unroll
@@ -510,7 +538,7 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_kernel(
             for (int w = 0; w < R / 16; ++w) acc[w] = Bf::mfma16(value_operand<R>(vt, 0, w, lane), pb, acc[w]);
         } else {
 #pragma unroll
-            for (int w = 0; w < RV / 16; ++w) acc[w] = Bf::mfma16(latent_operand<R>(kt, w, lane), pb, acc[w]);
+            for (int w = 0; w < RV / 16; ++w) acc[w] = Bf::mfma16(latent_operand<RV>(kt, w, lane), pb, acc[w]);
         }
         asm volatile("s_waitcnt lgkmcnt(0)" : : : "memory");   // the tile is free for the next loads
     }
@@ -527,46 +555,89 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_kernel(
         mine[lo * RS + RV + 1] = l;
     }
     __syncthreads();
-    for (int i = threadIdx.x; i < n_heads * vdim; i += 64 * WAVES) {
-        const int h = i / vdim, d = i - h * vdim;
-        float mm = kNegBig, lt = 0.f, at = 0.f;
+    // per head: what each wave's result counts (in place of its maximum), and what is known of the whole split
+    if (threadIdx.x < n_heads) {
+        const int h = threadIdx.x;
+        float* o[WAVES];
+        float mm = kNegBig, lt = 0.f;
 #pragma unroll
-        for (int w = 0; w < WAVES; ++w) mm = fmaxf(mm, reinterpret_cast<const float*>(s_raw + w * kWave)[h * RS + RV]);
+        for (int w = 0; w < WAVES; ++w) {
+            o[w] = reinterpret_cast<float*>(s_raw + w * kWave) + h * RS + RV;
+            mm = fmaxf(mm, o[w][0]);
+        }
+#pragma unroll
+        for (int w = 0; w < WAVES; ++w) {
+            o[w][0] = exp2_raw(o[w][0] - mm);
+            lt += o[w][1] * o[w][0];
+        }
+        if (splits == 1) {
+#pragma unroll
+            for (int w = 0; w < WAVES; ++w) o[w][0] /= lt;
+        } else {
+            float* dst = partial + (((int64_t)b * heads + h0 + h) * splits + sp) * (vdim + 4) + vdim;
+            dst[0] = mm;
+            dst[1] = lt;
+        }
+    }
+    __syncthreads();
+    const int quads = (vdim + 3) >> 2;
+    for (int i = threadIdx.x; i < n_heads * quads; i += 64 * WAVES) {
+        const int h = i / quads, d = (i - h * quads) * 4;
+        f32x4 at = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int w = 0; w < WAVES; ++w) {
             const float* o = reinterpret_cast<const float*>(s_raw + w * kWave) + h * RS;
-            const float f = exp2_raw(o[RV] - mm);
-            lt += o[RV + 1] * f;
-            at += o[d] * f;
+            const f32x4 v = *reinterpret_cast<const f32x4*>(o + d);
+            const float f = o[RV];
+#pragma unroll
+            for (int e = 0; e < 4; ++e) at[e] += v[e] * f;
         }
         const int64_t head = (int64_t)b * heads + h0 + h;
+        const float r[4] = {at[0], at[1], at[2], at[3]};
         if (splits == 1) {
-            Bf::store(out + head * vdim + d, at / lt);
+            uint16_t* dst = out + head * vdim + d;
+            if (vdim % 4 == 0) {
+                store_vec<Bf, 4>(dst, r);
+            } else {
+                for (int e = 0; e < 4; ++e)
+                    if (d + e < vdim) Bf::store(dst + e, r[e]);
+            }
         } else {
-            float* dst = partial + (head * splits + sp) * (vdim + 2);
-            dst[d] = at;
-            if (d == 0) {
-                dst[vdim] = mm;
-                dst[vdim + 1] = lt;
+            float* dst = partial + (head * splits + sp) * (vdim + 4) + d;
+            if (vdim % 4 == 0) {
+                *reinterpret_cast<f32x4*>(dst) = at;
+            } else {
+                for (int e = 0; e < 4; ++e)
+                    if (d + e < vdim) dst[e] = r[e];
             }
         }
     }
 }
 
+// One workgroup per head; `splits` is at most 64.
 __global__ __launch_bounds__(256) void attn_merge_kernel(const float* __restrict__ partial, uint16_t* __restrict__ out,
                                                          int vdim, int splits) {
+    __shared__ float s_f[64];
     const int64_t head = blockIdx.x;
-    const float* p = partial + head * splits * (vdim + 2);
-    float mm = kNegBig;
-    for (int s = 0; s < splits; ++s) mm = fmaxf(mm, p[s * (vdim + 2) + vdim]);
+    const float* p = partial + head * splits * (vdim + 4);
+    if (threadIdx.x < 64) {
+        const int s = min((int)threadIdx.x, splits - 1);
+        const bool live = (int)threadIdx.x < splits;
+        const float m = p[s * (vdim + 4) + vdim], l = p[s * (vdim + 4) + vdim + 1];
+        const float mm = wave_max(m), f = live ? exp2_raw(m - mm) : 0.f;   // lanes past the splits repeat the last
+        s_f[threadIdx.x] = f / wave_sum(l * f);
+    }
+    __syncthreads();
     for (int d = threadIdx.x; d < vdim; d += 256) {
-        float lt = 0.f, at = 0.f;
-        for (int s = 0; s < splits; ++s) {
-            const float f = exp2_raw(p[s * (vdim + 2) + vdim] - mm);
-            lt += p[s * (vdim + 2) + vdim + 1] * f;
-            at += p[s * (vdim + 2) + d] * f;
+        float at = 0.f;
+        for (int s0 = 0; s0 < splits; s0 += 8) {                   // eight loads in flight
+            float v[8];
+#pragma unroll
+            for (int u = 0; u < 8; ++u) v[u] = p[min(s0 + u, splits - 1) * (vdim + 4) + d];
+#pragma unroll
+            for (int u = 0; u < 8; ++u) at += v[u] * (s0 + u < splits ? s_f[s0 + u] : 0.f);
         }
-        Bf::store(out + head * vdim + d, at / lt);
+        Bf::store(out + head * vdim + d, at);
     }
 }
 
@@ -665,7 +736,7 @@ extern "C" size_t nqh_attention_decode_workspace_bytes(int64_t batch, int64_t he
                                                        int64_t max_context, int64_t chunk, int64_t window, int dtype) {
     if (batch <= 0 || heads <= 0 || kv_heads <= 0 || v_row <= 0 || !matrix_form(v_row, v_row, dtype)) return 0;
     const int splits = decode_splits(batch, heads, kv_heads, decode_waves((int)v_row), most_keys(max_context, chunk, window));
-    return splits > 1 ? (size_t)(batch * heads * splits * (v_row + 2)) * sizeof(float) : 0;
+    return splits > 1 ? (size_t)(batch * heads * splits * (v_row + 4)) * sizeof(float) : 0;
 }
 
 extern "C" int nqh_attention_decode(const void* q, const void* k_cache, const void* v_cache, const int32_t* block_table,
@@ -684,8 +755,8 @@ extern "C" int nqh_attention_decode(const void* q, const void* k_cache, const vo
             return fail(NQH_ERR_ARG, fn, "misaligned pointer");
         const int64_t max_context = block_size * max_blocks, head_tiles = cdiv(heads / kv_heads, 16);
         const int splits = decode_splits(batch, heads, kv_heads, decode_waves((int)v_row), most_keys(max_context, chunk, window));
-        const size_t need = splits > 1 ? (size_t)(batch * heads * splits * (vdim + 2)) * sizeof(float) : 0;
-        if (need && (!workspace || workspace_bytes < need || !aligned(workspace, 4)))
+        const size_t need = splits > 1 ? (size_t)(batch * heads * splits * (vdim + 4)) * sizeof(float) : 0;
+        if (need && (!workspace || workspace_bytes < need || !aligned(workspace, 16)))
             return fail(NQH_ERR_WORKSPACE, fn, "workspace of %zu bytes needed, %zu given", need, workspace ? workspace_bytes : 0);
         const int64_t groups = batch * kv_heads * head_tiles * splits;
         if (groups > kMaxI32 || batch * heads > kMaxI32) return fail(NQH_ERR_ARG, fn, "problem too large");
@@ -724,6 +795,11 @@ extern "C" int nqh_attention_decode(const void* q, const void* k_cache, const vo
         else if ((rr) == 32) { constexpr int RL = 512, R = 544; __VA_ARGS__; }                  \
         else { constexpr int RL = 512, R = 576; __VA_ARGS__; }                                  \
     } while (0)
+// Context splits: one workgroup per CU (that is what its LDS allows at the wide rows), at least a tile per wave.
+static int latent_splits(int64_t batch, int64_t heads, int64_t longest) {
+    const int64_t want = 256 / std::max<int64_t>(1, batch * cdiv(heads, 16));
+    return (int)std::max<int64_t>(1, std::min({want, longest / (32 * kLatentWaves), (int64_t)64}));
+}
 static bool latent_matrix_form(int64_t rot_at, int64_t row, int dtype) {
     return dtype == NQH_BF16 && (rot_at == 64 || rot_at == 128 || rot_at == 256 || rot_at == 512) &&
            (row - rot_at == 32 || row - rot_at == 64);
@@ -732,8 +808,8 @@ static bool latent_matrix_form(int64_t rot_at, int64_t row, int dtype) {
 extern "C" size_t nqh_latent_attention_decode_workspace_bytes(int64_t batch, int64_t heads, int64_t rank, int64_t rot_at,
                                                               int64_t row, int64_t max_context, int dtype) {
     if (batch <= 0 || heads <= 0 || rank <= 0 || !latent_matrix_form(rot_at, row, dtype)) return 0;
-    const int splits = decode_splits(batch, heads, 1, kLatentWaves, max_context);
-    return splits > 1 ? (size_t)(batch * heads * splits * (rank + 2)) * sizeof(float) : 0;
+    const int splits = latent_splits(batch, heads, max_context);
+    return splits > 1 ? (size_t)(batch * heads * splits * (rank + 4)) * sizeof(float) : 0;
 }
 
 extern "C" int nqh_latent_attention_decode(const void* q, const void* cache, const int32_t* block_table,
@@ -760,9 +836,9 @@ extern "C" int nqh_latent_attention_decode(const void* q, const void* cache, con
     }
     if (!aligned(q, 16) || !aligned(cache, 16)) return fail(NQH_ERR_ARG, fn, "misaligned pointer");
     const int64_t head_tiles = cdiv(heads, 16);
-    const int splits = decode_splits(batch, heads, 1, kLatentWaves, block_size * max_blocks);
-    const size_t need = splits > 1 ? (size_t)(batch * heads * splits * (rank + 2)) * sizeof(float) : 0;
-    if (need && (!workspace || workspace_bytes < need || !aligned(workspace, 4)))
+    const int splits = latent_splits(batch, heads, block_size * max_blocks);
+    const size_t need = splits > 1 ? (size_t)(batch * heads * splits * (rank + 4)) * sizeof(float) : 0;
+    if (need && (!workspace || workspace_bytes < need || !aligned(workspace, 16)))
         return fail(NQH_ERR_WORKSPACE, fn, "workspace of %zu bytes needed, %zu given", need, workspace ? workspace_bytes : 0);
     const int64_t groups = batch * head_tiles * splits;
     if (groups > kMaxI32 || batch * heads > kMaxI32) return fail(NQH_ERR_ARG, fn, "problem too large");
@@ -811,7 +887,7 @@ extern "C" int nqh_latent_attention_prefill(const void* q, const void* kv, int64
     else if (row == 128 && vdim <= 64) NQH_GO(128, 64, 64);
     else if (row == 128) NQH_GO(128, 128, 64);
     else if (row == 192 && vdim <= 64) NQH_GO(192, 64, 32);
-    else if (row == 192) NQH_GO(192, 128, 32);
+    else if (row == 192) NQH_GO(192, 128, 64);
     else if (vdim <= 128) NQH_GO(256, 128, 32);
     else NQH_GO(256, 256, 32);
 #undef NQH_GO

@@ -130,6 +130,10 @@ __device__ __forceinline__ float block_sum(float v, float* s) {
 
 __device__ __forceinline__ float sigmoid_f32(float z) { return 1.f / (1.f + expf(-z)); }
 __device__ __forceinline__ float silu_f32(float z) { return z / (1.f + expf(-z)); }
+// The same by the hardware's 2^x and reciprocal (about one ulp each), for kernels that the exact division would slow down.
+__device__ __forceinline__ float silu_quick(float z) {
+    return z * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(z * -1.4426950408889634f));
+}
 // sigmoid(z)^(1 / tau) = 2^(-(log2(1 + e^-|z|) + max(-z, 0) log2 e) / tau).  log(1 + x) as log(u) x / (u - 1) with
 // u = 1 + x rounded keeps its relative precision for small x (Goldberg, "What every computer scientist should know about
 // floating-point arithmetic", theorem 4).

@@ -68,8 +68,57 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(const typename T::elem* 
             for (int e = 0; e < V; ++e) a[e] += T::load(w + (int64_t)(c + e) * taps + k) * v[e];
         }
 #pragma unroll
-        for (int e = 0; e < V; ++e) a[e] = silu_f32(a[e]);
+        for (int e = 0; e < V; ++e) a[e] = silu_quick(a[e]);
         store_vec<T, V>(out + (int64_t)(pc.first + r0) * channels + c, a);
+    }
+}
+
+// Up to four taps: the weights and the rows that kConvRows tokens need are in registers before the first is used.
+constexpr int kConvRows = 8;
+template <typename T, int V>
+__global__ __launch_bounds__(256) void conv4_silu_kernel(const typename T::elem* __restrict__ x, int64_t x_stride,
+                                                         const typename T::elem* __restrict__ w,
+                                                         const typename T::elem* __restrict__ bias,
+                                                         const float* __restrict__ tail, const int32_t* __restrict__ pieces,
+                                                         typename T::elem* __restrict__ out, int channels, int taps) {
+    const Piece pc = load_piece_desc(pieces, blockIdx.y);
+    const int c = (blockIdx.x * 256 + threadIdx.x) * V, r0 = blockIdx.z * kConvRows;
+    if (c >= channels || r0 >= pc.rows) return;
+    float v[kConvRows + 3][V], wt[4][V], b[V];
+#pragma unroll
+    for (int j = 0; j < kConvRows + 3; ++j) {      // rows ahead of the sequence's tokens are replaced below
+        const int at = min(r0 + j - 3, pc.rows - 1);
+        load_vec<T, V>(x + (int64_t)max(pc.first + at, pc.index == 0 ? pc.first : 0) * x_stride + c, v[j]);
+    }
+    load_vec<T, V>(bias + c, b);
+#pragma unroll
+    for (int k = 0; k < 4; ++k)                    // tap k of four; the missing ones in front are zero
+#pragma unroll
+        for (int e = 0; e < V; ++e) {
+            const float f = T::load(w + (int64_t)(c + e) * taps + max(k - (4 - taps), 0));
+            wt[k][e] = k >= 4 - taps ? f : 0.f;
+        }
+    if (r0 == 0 && pc.index == 0) {
+#pragma unroll
+        for (int j = 0; j < 3; ++j) {
+            const int k = j - (4 - taps);          // place in the stored inputs
+#pragma unroll
+            for (int e = 0; e < V; ++e)
+                v[j][e] = k < 0 || pc.fresh ? 0.f : tail[((int64_t)pc.slot * (taps - 1) + k) * channels + c + e];
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < kConvRows; ++j) {
+        if (r0 + j >= pc.rows) return;
+        float a[V];
+#pragma unroll
+        for (int e = 0; e < V; ++e) {
+            a[e] = b[e];
+#pragma unroll
+            for (int k = 0; k < 4; ++k) a[e] += wt[k][e] * v[j + k][e];
+            a[e] = silu_quick(a[e]);
+        }
+        store_vec<T, V>(out + (int64_t)(pc.first + r0 + j) * channels + c, a);
     }
 }
 
@@ -96,55 +145,159 @@ __global__ __launch_bounds__(256) void conv_step_kernel(const typename T::elem* 
         }
         if (taps > 1) t[(int64_t)(taps - 2) * channels] = now;
     }
-    T::store(out + (int64_t)row * channels + c, live ? silu_f32(a) : 0.f);
+    T::store(out + (int64_t)row * channels + c, live ? silu_quick(a) : 0.f);
 }
 
 // ---- step sizes --------------------------------------------------------------------------------------------------------
-// dt [rows, channels] fp32.  Matrix cores: a wave takes 16 channels of 16 rows, the workgroup four times as many channels.
+// dt [rows, channels] fp32.  Matrix cores: the workgroup's four waves lie 2 x 2, a wave takes 16 CT channels of 16 RT rows and
+// has the next step's operands in flight.
+template <int CT, int RT>
 __global__ __launch_bounds__(256) void scan_dt_kernel(const uint16_t* __restrict__ low, int64_t low_stride,
                                                       const uint16_t* __restrict__ w, const uint16_t* __restrict__ bias,
                                                       float* __restrict__ dt, int rows, int channels, int rank) {
     const int lane = threadIdx.x & 63, lo = lane & 15, hi = lane >> 4, wave = threadIdx.x >> 6;
-    const int c0 = blockIdx.x * 64 + wave * 16;
-    const int64_t r0 = (int64_t)blockIdx.y * 64;
-    if (c0 >= channels) return;
-    const uint16_t* wr = w + (int64_t)min(c0 + lo, channels - 1) * rank;
-    const uint16_t* xr[4];
-    f32x4 acc[4];
+    const int c0 = blockIdx.x * 32 * CT + (wave & 1) * 16 * CT;
+    const int64_t r0 = (int64_t)blockIdx.y * 32 * RT + (wave >> 1) * 16 * RT;
+    if (c0 >= channels || r0 >= rows) return;
+    const uint16_t *wr[CT], *xr[RT];
+    f32x4 acc[CT][RT];
 #pragma unroll
-    for (int m = 0; m < 4; ++m) {
+    for (int i = 0; i < CT; ++i) wr[i] = w + (int64_t)min(c0 + 16 * i + lo, channels - 1) * rank;
+#pragma unroll
+    for (int m = 0; m < RT; ++m) {
         xr[m] = low + min(r0 + 16 * m + lo, (int64_t)rows - 1) * low_stride;
-        acc[m] = f32x4{0.f, 0.f, 0.f, 0.f};
-    }
-    for (int k0 = 0; k0 < rank; k0 += 32) {
-        const int k = k0 + 8 * hi, kc = min(k, rank - 8);
-        u32x4 a = *reinterpret_cast<const u32x4*>(wr + kc);
-        if (k >= rank) a = u32x4{0u, 0u, 0u, 0u};
 #pragma unroll
-        for (int m = 0; m < 4; ++m) {
-            u32x4 b = *reinterpret_cast<const u32x4*>(xr[m] + kc);
-            if (k >= rank) b = u32x4{0u, 0u, 0u, 0u};
-            acc[m] = Bf::mfma16(a, b, acc[m]);
+        for (int i = 0; i < CT; ++i) acc[i][m] = f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+    u32x4 a[2][CT], b[2][RT];
+    auto load = [&](u32x4 (&as)[CT], u32x4 (&bs)[RT], int k0) {
+        const int k = k0 + 8 * hi, kc = min(k, rank - 8);
+#pragma unroll
+        for (int i = 0; i < CT; ++i) as[i] = *reinterpret_cast<const u32x4*>(wr[i] + kc);
+#pragma unroll
+        for (int m = 0; m < RT; ++m) bs[m] = *reinterpret_cast<const u32x4*>(xr[m] + kc);
+    };
+    auto multiply = [&](const u32x4 (&as)[CT], u32x4 (&bs)[RT], int k0) {
+        if (k0 + 32 > rank) {                                     // the weights repeat past the end, the inputs are zero
+#pragma unroll
+            for (int m = 0; m < RT; ++m)
+                if (k0 + 8 * hi >= rank) bs[m] = u32x4{0u, 0u, 0u, 0u};
+        }
+#pragma unroll
+        for (int i = 0; i < CT; ++i)
+#pragma unroll
+            for (int m = 0; m < RT; ++m) acc[i][m] = Bf::mfma16(as[i], bs[m], acc[i][m]);
+    };
+    load(a[0], b[0], 0);
+    for (int k0 = 0; k0 < rank; k0 += 64) {
+        if (k0 + 32 < rank) load(a[1], b[1], k0 + 32);
+        multiply(a[0], b[0], k0);
+        if (k0 + 64 < rank) load(a[0], b[0], k0 + 64);
+        if (k0 + 32 < rank) multiply(a[1], b[1], k0 + 32);
+    }
+#pragma unroll
+    for (int i = 0; i < CT; ++i) {
+        const int c = c0 + 16 * i + 4 * hi;
+        float bv[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) bv[e] = Bf::to_f32(bias[min(c + e, channels - 1)]);
+#pragma unroll
+        for (int m = 0; m < RT; ++m) {
+            const int64_t r = r0 + 16 * m + lo;
+            if (r >= rows) continue;
+            float v[4];
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] = softplus_f32(acc[i][m][e] + bv[e]);
+            float* dst = dt + r * channels + c;
+            if (channels % 4 == 0) {
+                if (c < channels) store_vec<Fp, 4>(dst, v);
+            } else {
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    if (c + e < channels) dst[e] = v[e];
+            }
         }
     }
-    const int c = c0 + 4 * hi;
-    float b[4];
+}
+
+// The same for passes of many rows: 128 channels x 128 rows, operands through LDS in stages of 64 contraction elements,
+// double-buffered.  LDS rows are 128 bytes; 16-byte piece p of row r lies at position (p + r / 2) % 8, so that the 16 rows of
+// an operand read fall on different banks.
+#define NQH_GPTR(p) ((__attribute__((address_space(1))) void*)(p))
+#define NQH_LPTR(p) ((__attribute__((address_space(3))) void*)(p))
+__device__ const u32x4 g_zero_piece = {0u, 0u, 0u, 0u};   // what lies past the end of a row
+
+__global__ __launch_bounds__(256) void scan_dt_tile_kernel(const uint16_t* __restrict__ low, int64_t low_stride,
+                                                           const uint16_t* __restrict__ w, const uint16_t* __restrict__ bias,
+                                                           float* __restrict__ dt, int rows, int channels, int rank) {
+    constexpr int kTile = 128 * 128;                     // bytes of one operand's stage
+    __shared__ __attribute__((aligned(1024))) unsigned char s_mem[4 * kTile];      // [buffer][weights | rows]
+    const int lane = threadIdx.x & 63, lo = lane & 15, hi = lane >> 4;
+    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int c0 = blockIdx.x * 128, wc = (wave & 1) * 64, wr = (wave >> 1) * 64;
+    const int64_t r0 = (int64_t)blockIdx.y * 128;
+    const uint16_t *w_src[4], *x_src[4];
+    int k_src[4];
 #pragma unroll
-    for (int e = 0; e < 4; ++e) b[e] = Bf::to_f32(bias[min(c + e, channels - 1)]);
+    for (int i = 0; i < 4; ++i) {
+        const int n = (i * 4 + wave) * 64 + lane, row = n >> 3;
+        k_src[i] = 8 * (((n & 7) - (row >> 1)) & 7);
+        w_src[i] = w + (int64_t)min(c0 + row, channels - 1) * rank;
+        x_src[i] = low + min(r0 + row, (int64_t)rows - 1) * low_stride;
+    }
+    auto stage = [&](int k0, int buf) {
+        unsigned char* base = s_mem + buf * 2 * kTile + wave * 1024;
 #pragma unroll
-    for (int m = 0; m < 4; ++m) {
-        const int64_t r = r0 + 16 * m + lo;
-        if (r >= rows) continue;
-        float v[4];
+        for (int i = 0; i < 4; ++i) {
+            const int k = k0 + k_src[i];
+            const void* a = k < rank ? (const void*)(w_src[i] + k) : (const void*)&g_zero_piece;
+            const void* b = k < rank ? (const void*)(x_src[i] + k) : (const void*)&g_zero_piece;
+            __builtin_amdgcn_global_load_lds(NQH_GPTR(a), NQH_LPTR(base + i * 4096), 16, 0, 0);
+            __builtin_amdgcn_global_load_lds(NQH_GPTR(b), NQH_LPTR(base + kTile + i * 4096), 16, 0, 0);
+        }
+    };
+    f32x4 acc[4][4];
 #pragma unroll
-        for (int e = 0; e < 4; ++e) v[e] = softplus_f32(acc[m][e] + b[e]);
-        float* dst = dt + r * channels + c;
-        if (channels % 4 == 0) {
-            if (c < channels) store_vec<Fp, 4>(dst, v);
-        } else {
+    for (int i = 0; i < 4; ++i)
 #pragma unroll
-            for (int e = 0; e < 4; ++e)
-                if (c + e < channels) dst[e] = v[e];
+        for (int m = 0; m < 4; ++m) acc[i][m] = f32x4{0.f, 0.f, 0.f, 0.f};
+    stage(0, 0);
+    int buf = 0;
+    for (int k0 = 0; k0 < rank; k0 += 64) {
+        __builtin_amdgcn_s_waitcnt(0x0F70);              // this wave's part of the stage has landed
+        __syncthreads();
+        if (k0 + 64 < rank) stage(k0 + 64, buf ^ 1);
+        const unsigned char* base = s_mem + buf * 2 * kTile;
+#pragma unroll
+        for (int s = 0; s < 2; ++s) {
+            u32x4 a[4], b[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int ra = wc + 16 * i + lo, rb = wr + 16 * i + lo;
+                a[i] = *reinterpret_cast<const u32x4*>(base + ra * 128 + ((4 * s + hi + (ra >> 1)) & 7) * 16);
+                b[i] = *reinterpret_cast<const u32x4*>(base + kTile + rb * 128 + ((4 * s + hi + (rb >> 1)) & 7) * 16);
+            }
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int m = 0; m < 4; ++m) acc[i][m] = Bf::mfma16(a[i], b[m], acc[i][m]);
+        }
+        buf ^= 1;
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int c = c0 + wc + 16 * i + 4 * hi;
+        float bv[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) bv[e] = Bf::to_f32(bias[min(c + e, channels - 1)]);
+#pragma unroll
+        for (int m = 0; m < 4; ++m) {
+            const int64_t r = r0 + wr + 16 * m + lo;
+            if (r >= rows || c >= channels) continue;
+            float v[4];
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] = softplus_f32(acc[i][m][e] + bv[e]);
+            store_vec<Fp, 4>(dt + r * channels + c, v);  // the number of channels is a multiple of 4
         }
     }
 }
@@ -256,7 +409,7 @@ __global__ __launch_bounds__(256) void scan_piece_kernel(
 #pragma unroll
                 for (int o = 1; o < LPC; o <<= 1) y += __shfl_xor(y, o);
                 if (sub == 0 && live && t0 + u <= last)
-                    T::store(out + (int64_t)(pc.first + t0 + u) * channels + c, (y + D * xc[u]) * silu_f32(zc[u]));
+                    T::store(out + (int64_t)(pc.first + t0 + u) * channels + c, (y + D * xc[u]) * silu_quick(zc[u]));
             }
         }
         buf ^= 1;
@@ -301,9 +454,20 @@ __global__ __launch_bounds__(256) void scan_chain_kernel(const float* __restrict
     float S = pc.fresh ? 0.f : state[pc.slot * size + at];
     const int64_t p0 = blockIdx.z;
     ws_state[p0 * size + at] = S;
-    for (int p = 0; p < pc.count - 1; ++p) {
-        S = __builtin_amdgcn_exp2f(A * ws_dt[(p0 + p) * channels + c]) * S + ws_state[(p0 + p + 1) * size + at];
-        ws_state[(p0 + p + 1) * size + at] = S;
+    for (int p = 0; p < pc.count - 1; p += 8) {          // eight pieces' operands in flight
+        float d[8], v[8];
+#pragma unroll
+        for (int u = 0; u < 8; ++u) {
+            const int64_t q = p0 + min(p + u, pc.count - 2);
+            d[u] = ws_dt[q * channels + c];
+            v[u] = ws_state[(q + 1) * size + at];
+        }
+#pragma unroll
+        for (int u = 0; u < 8; ++u) {
+            if (p + u >= pc.count - 1) break;
+            S = __builtin_amdgcn_exp2f(A * d[u]) * S + v[u];
+            ws_state[(p0 + p + u + 1) * size + at] = S;
+        }
     }
 }
 
@@ -349,7 +513,7 @@ __global__ __launch_bounds__(256) void scan_step_kernel(
     __syncthreads();
     if (wave == 0 && cw < channels) {
         y = s_y[0][lane] + s_y[1][lane] + s_y[2][lane] + s_y[3][lane] + T::load(d_skip + c) * xv;
-        T::store(out + (int64_t)row * channels + c, ok ? y * silu_f32(T::load(z + row * z_stride + c)) : 0.f);
+        T::store(out + (int64_t)row * channels + c, ok ? y * silu_quick(T::load(z + row * z_stride + c)) : 0.f);
     }
 }
 
@@ -373,11 +537,9 @@ int check_scan(const char* fn, int64_t channels, int64_t states, int64_t taps, i
 using namespace nqh;
 
 extern "C" int64_t nqh_scan_piece_rows(int64_t rows, int64_t channels, int64_t states) {
-    // about 2048 workgroups
+    // Four workgroups per CU keep the vector ALU busy; more pieces than that only cost, each but a sequence's last runs twice.
     const int64_t groups = cdiv(channels, 256 / lanes_per_channel(states));
-    const int64_t want = cdiv(rows * groups, 2048);
-    int64_t size = kMinPiece;
-    while (size < want && size < 2048) size *= 2;
+    const int64_t size = std::max<int64_t>(kMinPiece, cdiv(cdiv(rows * groups, 1024), 32) * 32);
     return size;
 }
 extern "C" size_t nqh_scan_workspace_bytes(int64_t num_pieces, int64_t channels, int64_t states) {
@@ -395,15 +557,17 @@ extern "C" int nqh_conv_silu(const void* x, int64_t x_stride, const void* weight
     if (num_pieces <= 0 || num_pieces > 65535 || longest <= 0 || cdiv(longest, 8) > 65535 || x_stride < channels)
         return fail(NQH_ERR_ARG, fn, "1 to 65535 pieces, and x rows at least as wide as the channels");
     (void)hipGetLastError();
-#define NQH_GO(V)                                                                                                       \
-    conv_silu_kernel<T, V><<<dim3((unsigned)cdiv(channels, 256 * V), (unsigned)num_pieces, (unsigned)cdiv(longest, 8)),  \
-                             dim3(256), 0, (hipStream_t)stream>>>((const E*)x, x_stride, (const E*)weight, (const E*)bias, \
-                                                                  tail, pieces, (E*)out, (int)channels, (int)taps)
+#define NQH_GO(KERNEL, V)                                                                                                 \
+    KERNEL<T, V><<<dim3((unsigned)cdiv(channels, 256 * V), (unsigned)num_pieces, (unsigned)cdiv(longest, 8)), dim3(256), 0, \
+                   (hipStream_t)stream>>>((const E*)x, x_stride, (const E*)weight, (const E*)bias, tail, pieces, (E*)out,   \
+                                          (int)channels, (int)taps)
     NQH_WITH_TYPE(dtype, {
         using E = typename T::elem;
-        const bool vec = channels % 4 == 0 && x_stride % 4 == 0 && aligned(x, 4 * sizeof(E)) && aligned(out, 4 * sizeof(E));
-        if (vec) NQH_GO(4);
-        else NQH_GO(1);
+        constexpr int V = 16 / sizeof(E);
+        const bool vec = channels % V == 0 && x_stride % V == 0 && aligned(x, 16) && aligned(bias, 16) && aligned(out, 16);
+        if (taps <= 4 && vec) NQH_GO(conv4_silu_kernel, V);
+        else if (vec) NQH_GO(conv_silu_kernel, V);
+        else NQH_GO(conv_silu_kernel, 1);
     });
 #undef NQH_GO
     return launched(fn);
@@ -439,12 +603,20 @@ extern "C" int nqh_scan_dt(const void* low, int64_t low_stride, const void* weig
         return fail(NQH_ERR_ARG, fn, "sizes must be positive 31-bit counts and the rows as wide as the rank");
     const bool matrix = dtype == NQH_BF16 && rank % 8 == 0 && low_stride % 8 == 0 && aligned(low, 16) && aligned(weight, 16) &&
                         aligned(dt, 16);
-    if (cdiv(rows, 64) > 65535 || (!matrix && rows > 65535)) return fail(NQH_ERR_UNSUPPORTED, fn, "too many rows");
+    if (cdiv(rows, 128) > 65535 || (!matrix && rows > 65535)) return fail(NQH_ERR_UNSUPPORTED, fn, "too many rows");
     (void)hipGetLastError();
     if (matrix) {
-        scan_dt_kernel<<<dim3((unsigned)cdiv(channels, 64), (unsigned)cdiv(rows, 64)), dim3(256), 0, (hipStream_t)stream>>>(
-            (const uint16_t*)low, low_stride, (const uint16_t*)weight, (const uint16_t*)bias, dt, (int)rows, (int)channels,
-            (int)rank);
+#define NQH_GO(CT, RT)                                                                                                    \
+    scan_dt_kernel<CT, RT><<<dim3((unsigned)cdiv(channels, 32 * CT), (unsigned)cdiv(rows, 32 * RT)), dim3(256), 0,         \
+                             (hipStream_t)stream>>>((const uint16_t*)low, low_stride, (const uint16_t*)weight,             \
+                                                    (const uint16_t*)bias, dt, (int)rows, (int)channels, (int)rank)
+        if (rows <= 64) NQH_GO(1, 1);
+        else if (channels % 4 != 0 || rows < 512) NQH_GO(2, 4);
+        else
+            scan_dt_tile_kernel<<<dim3((unsigned)cdiv(channels, 128), (unsigned)cdiv(rows, 128)), dim3(256), 0,
+                                  (hipStream_t)stream>>>((const uint16_t*)low, low_stride, (const uint16_t*)weight,
+                                                         (const uint16_t*)bias, dt, (int)rows, (int)channels, (int)rank);
+#undef NQH_GO
         return launched(fn);
     }
     NQH_WITH_TYPE(dtype, {

@@ -411,6 +411,15 @@ def test_selective_scan_prefill_portions_and_decode(dtype, T, C, N, rank, taps):
         assert torch.equal(tail[2].cpu().double(), tail_want)
 
 
+@pytest.mark.parametrize("rows,channels,rank", [(512, 128, 64), (700, 200, 72), (1030, 36, 8), (513, 300, 128), (600, 30, 24)])
+def test_scan_step_sizes_of_long_passes(rows, channels, rank):
+    print(f"scan_dt {rows}x{channels} rank {rank}", flush=True)
+    low, up = rand(rows, rank + 16, seed=1, dtype=torch.bfloat16), rand(channels, rank, seed=2, dtype=torch.bfloat16)
+    b = rand(channels, seed=3, dtype=torch.bfloat16)
+    got = ops.scan_dt(low.cuda()[:, :rank], up.cuda(), b.cuda())
+    close(got, o.softplus(low[:, :rank].double() @ up.double().T + b.double()), torch.float32)
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 def test_one_state_entry_lives_on(dtype):
     """A single token writes the state and slow decays keep it: the read-out far behind it, over pieces, portions and steps,
