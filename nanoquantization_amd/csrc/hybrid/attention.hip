@@ -3,8 +3,8 @@
 // [block][kv head][token][row], a row being a head's dim (vdim) elements and zero padding.
 //   attn_tile_kernel     prompts in bf16: 128 query tokens of one head per workgroup, both products on the matrix cores; keys
 //                        and values from the cache, or of latent attention expanded per head (DENSE)
-//   attn_decode_kernel   decode in bf16: the query heads of a kv head are the columns of the same products; for latent
-//                        attention one cache row is key and value of all heads
+//   attn_decode_kernel   decode in bf16: the query heads of a kv head are the columns of the same products
+//   latent_decode_kernel decode of latent attention in bf16: one cache row is key and value of all heads
 //   attn_rows_kernel     any sizes, both element types: one wave per (query token, head), arithmetic on the vector ALU
 #include <algorithm>
 
@@ -153,12 +153,22 @@ __device__ __forceinline__ u32x4 value_operand(const unsigned char* v_tile, int 
     return u32x4{ua[0], ua[1], ub[0], ub[1]};
 }
 
-// The same from rows in the layout of K tiles (a row that is key and value).
+// Rows of latents.  One of 512 elements is a load-to-LDS of its own, so rows can lie 1040 bytes apart instead of being
+// rotated: the places of all operands of a lane then differ by constants.
+template <int R>
+struct LatentLayout {
+    static constexpr int kLoadBytes = R == 512 ? 1040 : 1024, kTile = 32 * R * 2 / 1024 * kLoadBytes;
+    static __device__ __forceinline__ int source(int row, int pos) { return R == 512 ? 8 * pos : RowLayout<R>::k_source(row, pos); }
+    static __device__ __forceinline__ int at(int row, int piece) {
+        return R == 512 ? row * kLoadBytes + 16 * piece : RowLayout<R>::k_at(row, piece);
+    }
+};
+// value_operand from such rows.
 template <int R>
 __device__ __forceinline__ u32x4 latent_operand(const unsigned char* tile, int w, int lane) {
-    const int lo = lane & 15, hi = lane >> 4, row = 4 * hi + (lo >> 2), piece = 2 * w + ((lo & 3) >> 1), half = (lo & 1) * 8;
-    const unsigned char* p0 = tile + RowLayout<R>::k_at(row, piece) + half;
-    const unsigned char* p1 = tile + RowLayout<R>::k_at(row + 16, piece) + half;
+    const int lo = lane & 15, hi = lane >> 4, row = 4 * hi + (lo >> 2), sub = (lo & 3) >> 1, half = (lo & 1) * 8;
+    const unsigned char* p0 = tile + LatentLayout<R>::at(row, 2 * w + sub) + half;
+    const unsigned char* p1 = tile + LatentLayout<R>::at(row + 16, 2 * w + sub) + half;
     const s16x4 a = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)p0);
     const s16x4 b = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)p1);
     const u32x2 ua = __builtin_bit_cast(u32x2, a), ub = __builtin_bit_cast(u32x2, b);
@@ -399,22 +409,18 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
 }
 
 // Decode attention.  Workgroup = (sequence, kv head, 16 of its query heads, context split); a wave takes tiles of 32 keys
-// through its own part of LDS, no barriers until the merge.  RL > 0: latent attention, the first RL elements of a key row are
-// the value row; they and the rest lie in two tiles whose row widths are powers of two, so that a load-to-LDS takes whole
-// rows and needs next to no address arithmetic.
-template <int R, int WAVES, int RL>
+// through its own part of LDS, no barriers until the merge.
+template <int R, int WAVES>
 __global__ __launch_bounds__(64 * WAVES) void attn_decode_kernel(
     const uint16_t* __restrict__ q, const uint16_t* __restrict__ k_cache, const uint16_t* __restrict__ v_cache,
     const int32_t* __restrict__ block_table, const int32_t* __restrict__ context_lens, const uint16_t* __restrict__ sink,
     uint16_t* __restrict__ out, float* __restrict__ partial, int heads, int kv_heads, int vdim, int block_size, int max_blocks,
     int num_blocks, int chunk, int window, float scale, int splits, int head_tiles) {
     using L = RowLayout<R>;
-    using LL = RowLayout<RL == 0 ? 32 : RL>;
-    using LR = RowLayout<RL == 0 ? 32 : R - RL>;
-    constexpr int RV = RL > 0 ? RL : R, RS = RV + 4;      // value elements, width of a result row
+    constexpr int RS = R + 4;                             // width of a result row
     constexpr int TT = 32, kBytes = TT * R * 2, kLoads = kBytes / 1024;
-    constexpr int kWave = RL > 0 ? kBytes : 2 * kBytes + 1024;
-    static_assert(RV <= R && 16 * RS * 4 <= kWave && WAVES * kWave <= 160 * 1024, "the per-wave results reuse the wave's tiles");
+    constexpr int kWave = 2 * kBytes + 1024;
+    static_assert(16 * RS * 4 <= kWave, "the per-wave results reuse the wave's tiles");
     __shared__ __attribute__((aligned(1024))) unsigned char s_raw[WAVES * kWave];
     const int sp = blockIdx.x % splits, ht = blockIdx.x / splits % head_tiles;
     const int g = blockIdx.x / (splits * head_tiles) % kv_heads, b = blockIdx.x / (splits * head_tiles * kv_heads);
@@ -441,9 +447,9 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_kernel(
         m = Bf::to_f32(sink[h0 + min(lo, n_heads - 1)]) * kLog2e;
         l = hi == 0 ? 1.f : 0.f;
     }
-    f32x4 acc[RV / 16];
+    f32x4 acc[R / 16];
 #pragma unroll
-    for (int w = 0; w < RV / 16; ++w) acc[w] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int w = 0; w < R / 16; ++w) acc[w] = f32x4{0.f, 0.f, 0.f, 0.f};
     const int32_t* table = block_table + (int64_t)b * max_blocks;
     for (int tb = t0 + wave * TT; tb < t1; tb += WAVES * TT) {
         // the cache row of key tb + lane % 32 (past the split's end the last key stands in)
@@ -451,59 +457,29 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_kernel(
         int blk = table[j / block_size];
         blk = blk < 0 ? 0 : (blk >= num_blocks ? num_blocks - 1 : blk);
         const int my_row = (blk * kv_heads + g) * block_size + j % block_size;
-        if constexpr (RL == 0) {
 #pragma unroll
-            for (int i = 0; i < kLoads; ++i) {
-                const int n = i * 64 + lane, row = n / L::kPieces;
-                const int64_t base = (int64_t)__shfl(my_row, row) * R;
-                __builtin_amdgcn_global_load_lds(NQH_GPTR(k_cache + base + L::k_source(row, n % L::kPieces)),
-                                                 NQH_LPTR(kt + i * 1024), 16, 0, 0);
-            }
-#pragma unroll
-            for (int i = 0; i < kLoads; ++i) {
-                const int n = i * 64 + lane, row = n / L::kPieces;
-                const int64_t base = (int64_t)__shfl(my_row, row) * R;
-                __builtin_amdgcn_global_load_lds(NQH_GPTR(v_cache + base + L::v_source(row, n % L::kPieces)),
-                                                 NQH_LPTR(vt + i * 1024), 16, 0, 0);
-            }
-            // a wave's loads return in order: with at most the V tile's outstanding, the K tile has landed
-            asm volatile("s_waitcnt vmcnt(%0)" : : "n"(kLoads) : "memory");
-        } else {
-#pragma unroll
-            for (int i = 0; i < LL::kPieces / 2; ++i) {
-                const int n = i * 64 + lane, row = n / LL::kPieces;
-                const int64_t base = (int64_t)(LL::kPieces == 64 ? __builtin_amdgcn_readlane(my_row, i) : __shfl(my_row, row)) * R;
-                __builtin_amdgcn_global_load_lds(NQH_GPTR(k_cache + base + LL::k_source(row, n % LL::kPieces)),
-                                                 NQH_LPTR(kt + i * 1024), 16, 0, 0);
-            }
-#pragma unroll
-            for (int i = 0; i < LR::kPieces / 2; ++i) {
-                const int n = i * 64 + lane, row = n / LR::kPieces;
-                const int64_t base = (int64_t)__shfl(my_row, row) * R + RL;
-                __builtin_amdgcn_global_load_lds(NQH_GPTR(k_cache + base + LR::k_source(row, n % LR::kPieces)),
-                                                 NQH_LPTR(kt + TT * RL * 2 + i * 1024), 16, 0, 0);
-            }
-            asm volatile("s_waitcnt vmcnt(0)" : : : "memory");
+        for (int i = 0; i < kLoads; ++i) {
+            const int n = i * 64 + lane, row = n / L::kPieces;
+            const int64_t base = (int64_t)__shfl(my_row, row) * R;
+            __builtin_amdgcn_global_load_lds(NQH_GPTR(k_cache + base + L::k_source(row, n % L::kPieces)),
+                                             NQH_LPTR(kt + i * 1024), 16, 0, 0);
         }
+#pragma unroll
+        for (int i = 0; i < kLoads; ++i) {
+            const int n = i * 64 + lane, row = n / L::kPieces;
+            const int64_t base = (int64_t)__shfl(my_row, row) * R;
+            __builtin_amdgcn_global_load_lds(NQH_GPTR(v_cache + base + L::v_source(row, n % L::kPieces)),
+                                             NQH_LPTR(vt + i * 1024), 16, 0, 0);
+        }
+        // a wave's loads return in order: with at most the V tile's outstanding, the K tile has landed
+        asm volatile("s_waitcnt vmcnt(%0)" : : "n"(kLoads) : "memory");
         f32x4 st[2];
         st[0] = st[1] = f32x4{0.f, 0.f, 0.f, 0.f};
-        if constexpr (RL == 0) {
 #pragma unroll
-            for (int a = 0; a < 2; ++a)
-#pragma unroll
-                for (int s = 0; s < R / 32; ++s)
-                    st[a] = Bf::mfma16(*reinterpret_cast<const u32x4*>(kt + L::k_at(16 * a + lo, 4 * s + hi)), bq[s], st[a]);
-        } else {
+        for (int a = 0; a < 2; ++a)
 #pragma unroll
             for (int s = 0; s < R / 32; ++s)
-#pragma unroll
-                for (int a = 0; a < 2; ++a) {
-                    const int row = 16 * a + lo;
-                    const unsigned char* p = s < RL / 32 ? kt + LL::k_at(row, 4 * s + hi)
-                                                         : kt + TT * RL * 2 + LR::k_at(row, 4 * (s - RL / 32) + hi);
-                    st[a] = Bf::mfma16(*reinterpret_cast<const u32x4*>(p), bq[s], st[a]);
-                }
-        }
+                st[a] = Bf::mfma16(*reinterpret_cast<const u32x4*>(kt + L::k_at(16 * a + lo, 4 * s + hi)), bq[s], st[a]);
         float mx = kNegBig;
 #pragma unroll
         for (int a = 0; a < 2; ++a)
@@ -529,17 +505,12 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_kernel(
         const u32x4 pb = u32x4{Bf::pack2(p[0][0], p[0][1]), Bf::pack2(p[0][2], p[0][3]), Bf::pack2(p[1][0], p[1][1]),
                                Bf::pack2(p[1][2], p[1][3])};
 #pragma unroll
-        for (int w = 0; w < RV / 16; ++w)
+        for (int w = 0; w < R / 16; ++w)
 #pragma unroll
             for (int r = 0; r < 4; ++r) acc[w][r] *= f;
-        if constexpr (RL == 0) {
-            asm volatile("s_waitcnt vmcnt(0)" : : : "memory");
+        asm volatile("s_waitcnt vmcnt(0)" : : : "memory");
 #pragma unroll
-            for (int w = 0; w < R / 16; ++w) acc[w] = Bf::mfma16(value_operand<R>(vt, 0, w, lane), pb, acc[w]);
-        } else {
-#pragma unroll
-            for (int w = 0; w < RV / 16; ++w) acc[w] = Bf::mfma16(latent_operand<RV>(kt, w, lane), pb, acc[w]);
-        }
+        for (int w = 0; w < R / 16; ++w) acc[w] = Bf::mfma16(value_operand<R>(vt, 0, w, lane), pb, acc[w]);
         asm volatile("s_waitcnt lgkmcnt(0)" : : : "memory");   // the tile is free for the next loads
     }
     l += __shfl_xor(l, 16);
@@ -547,12 +518,12 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_kernel(
     // per-wave results [head][RS] over the wave's own tiles, then merged over the waves
     float* mine = reinterpret_cast<float*>(kt);
 #pragma unroll
-    for (int w = 0; w < RV / 16; ++w)
+    for (int w = 0; w < R / 16; ++w)
 #pragma unroll
         for (int r = 0; r < 4; ++r) mine[lo * RS + 16 * w + 4 * hi + r] = acc[w][r];
     if (hi == 0) {
-        mine[lo * RS + RV] = m;
-        mine[lo * RS + RV + 1] = l;
+        mine[lo * RS + R] = m;
+        mine[lo * RS + R + 1] = l;
     }
     __syncthreads();
     // per head: what each wave's result counts (in place of its maximum), and what is known of the whole split
@@ -562,7 +533,7 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_kernel(
         float mm = kNegBig, lt = 0.f;
 #pragma unroll
         for (int w = 0; w < WAVES; ++w) {
-            o[w] = reinterpret_cast<float*>(s_raw + w * kWave) + h * RS + RV;
+            o[w] = reinterpret_cast<float*>(s_raw + w * kWave) + h * RS + R;
             mm = fmaxf(mm, o[w][0]);
         }
 #pragma unroll
@@ -588,7 +559,7 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_kernel(
         for (int w = 0; w < WAVES; ++w) {
             const float* o = reinterpret_cast<const float*>(s_raw + w * kWave) + h * RS;
             const f32x4 v = *reinterpret_cast<const f32x4*>(o + d);
-            const float f = o[RV];
+            const float f = o[R];
 #pragma unroll
             for (int e = 0; e < 4; ++e) at[e] += v[e] * f;
         }
@@ -614,31 +585,183 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_kernel(
     }
 }
 
-// One workgroup per head; `splits` is at most 64.
-__global__ __launch_bounds__(256) void attn_merge_kernel(const float* __restrict__ partial, uint16_t* __restrict__ out,
+// Decode attention over latent rows of R elements, the first RL of which are the value.  Workgroup = (sequence, 16 HT heads,
+// context split): tiles of 32 keys, double-buffered, that all four waves read; a wave has one tile of 16 heads and a part of
+// the value elements, so nothing is merged between waves (those that share heads repeat the scores).  Latents and rotated
+// parts lie in two LDS tiles whose row widths are powers of two: a load-to-LDS takes whole rows and needs next to no address
+// arithmetic.
+template <int RL, int R, int HT>
+__global__ __launch_bounds__(256, 2) void latent_decode_kernel(
+    const uint16_t* __restrict__ q, const uint16_t* __restrict__ cache, const int32_t* __restrict__ block_table,
+    const int32_t* __restrict__ context_lens, uint16_t* __restrict__ out, float* __restrict__ partial, int heads, int rank,
+    int block_size, int max_blocks, int num_blocks, float scale, int splits, int head_groups) {
+    using LL = LatentLayout<RL>;
+    using LR = LatentLayout<R - RL>;
+    constexpr int TT = 32, kRot = LL::kTile, kBuffer = kRot + LR::kTile, kLoads = RL / 64, kPieces = RL / 8, rPieces = (R - RL) / 8;
+    constexpr int kParts = 4 / HT, kWindows = RL / 16 / kParts;
+    static_assert(2 * kBuffer <= 80 * 1024, "two workgroups per CU");
+    __shared__ __attribute__((aligned(1024))) unsigned char s_mem[2 * kBuffer];
+    const int sp = blockIdx.x % splits, hg = blockIdx.x / splits % head_groups, b = blockIdx.x / (splits * head_groups);
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int lo = lane & 15, hi = lane >> 4, part = wave / HT;
+    const int h0 = hg * 16 * HT + wave % HT * 16, head = min(h0 + lo, heads - 1);   // columns past the heads repeat the last
+    int ctx = context_lens[b];
+    ctx = ctx < 1 ? 1 : (ctx > max_blocks * block_size ? max_blocks * block_size : ctx);
+    const int tiles = (ctx + TT - 1) / TT;               // dealt evenly
+    const int t0 = (int)((int64_t)tiles * sp / splits) * TT, t1 = min(ctx, (int)((int64_t)tiles * (sp + 1) / splits) * TT);
+    const int32_t* table = block_table + (int64_t)b * max_blocks;
+    u32x4 bq[R / 32];
+#pragma unroll
+    for (int s = 0; s < R / 32; ++s)
+        bq[s] = *reinterpret_cast<const u32x4*>(q + ((int64_t)b * heads + head) * R + 32 * s + 8 * hi);
+    // the cache row of key tb + lane % 32 (past the split's end the last key stands in); the block number is fetched ahead
+    int next_block = 0;
+    auto key_of = [&](int tb) { return max(min(tb + (lane & 31), t1 - 1), 0); };
+    auto fetch_block = [&](int tb) { next_block = table[key_of(tb) / block_size]; };
+    auto stage = [&](int tb, int buf) {
+        const int blk = next_block < 0 ? 0 : (next_block >= num_blocks ? num_blocks - 1 : next_block);
+        const int my_row = blk * block_size + key_of(tb) % block_size;
+        unsigned char* base = s_mem + buf * kBuffer;
+        // every shuffle comes before the first load: the compiler has LDS instructions wait for loads-to-LDS
+        int rows[kLoads];
+#pragma unroll
+        for (int i = 0; i < kLoads; ++i) {                          // a wave brings eight rows
+            const int at = wave * kLoads + i;
+            rows[i] = kPieces == 64 ? __builtin_amdgcn_readlane(my_row, at) : __shfl(my_row, (at * 64 + lane) / kPieces);
+        }
+        const int rn = wave * 64 + lane, rot_row = __shfl(my_row, min(rn / rPieces, TT - 1));
+#pragma unroll
+        for (int i = 0; i < kLoads; ++i) {
+            const int at = wave * kLoads + i, n = at * 64 + lane;
+            __builtin_amdgcn_global_load_lds(NQH_GPTR(cache + (int64_t)rows[i] * R + LL::source(n / kPieces, n % kPieces)),
+                                             NQH_LPTR(base + at * LL::kLoadBytes), 16, 0, 0);
+        }
+        if (wave < rPieces / 2)                                     // 32 x 32 elements are two loads, 32 x 64 four
+            __builtin_amdgcn_global_load_lds(NQH_GPTR(cache + (int64_t)rot_row * R + RL + LR::source(rn / rPieces, rn % rPieces)),
+                                             NQH_LPTR(base + kRot + wave * 1024), 16, 0, 0);
+    };
+    const float sc = scale * kLog2e;
+    float m = kNegBig, l = 0.f;
+    f32x4 acc[kWindows];
+#pragma unroll
+    for (int w = 0; w < kWindows; ++w) acc[w] = f32x4{0.f, 0.f, 0.f, 0.f};
+    fetch_block(t0);
+    if (t0 < t1) stage(t0, 0);
+    fetch_block(t0 + TT);
+    int buf = 0;
+    for (int tb = t0; tb < t1; tb += TT) {
+        __builtin_amdgcn_s_waitcnt(0x0F70);   // this wave's part of the tile has landed
+        __syncthreads();
+        if (tb + TT < t1) {
+            stage(tb + TT, buf ^ 1);
+            fetch_block(tb + 2 * TT);
+        }
+        const unsigned char* tile = s_mem + buf * kBuffer;
+        f32x4 st[2];
+        st[0] = st[1] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int s = 0; s < R / 32; ++s)
+#pragma unroll
+            for (int a = 0; a < 2; ++a) {
+                const int row = 16 * a + lo;
+                const unsigned char* p = s < RL / 32 ? tile + LL::at(row, 4 * s + hi) : tile + kRot + LR::at(row, 4 * (s - RL / 32) + hi);
+                st[a] = Bf::mfma16(*reinterpret_cast<const u32x4*>(p), bq[s], st[a]);
+            }
+        float mx = kNegBig;
+#pragma unroll
+        for (int a = 0; a < 2; ++a)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                st[a][r] = tb + 16 * a + 4 * hi + r < t1 ? st[a][r] * sc : -__builtin_inff();
+                mx = fmaxf(mx, st[a][r]);
+            }
+        mx = fmaxf(mx, __shfl_xor(mx, 16));
+        mx = fmaxf(mx, __shfl_xor(mx, 32));
+        const float mn = fmaxf(m, mx);
+        if (__any(mn > m)) {
+            const float f = exp2_raw(m - mn);
+            m = mn;
+            l *= f;
+#pragma unroll
+            for (int w = 0; w < kWindows; ++w)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) acc[w][r] *= f;
+        }
+        float p[2][4];
+#pragma unroll
+        for (int a = 0; a < 2; ++a)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                p[a][r] = exp2_raw(st[a][r] - mn);
+                l += p[a][r];
+            }
+        const u32x4 pb = u32x4{Bf::pack2(p[0][0], p[0][1]), Bf::pack2(p[0][2], p[0][3]), Bf::pack2(p[1][0], p[1][1]),
+                               Bf::pack2(p[1][2], p[1][3])};
+#pragma unroll
+        for (int w = 0; w < kWindows; ++w)
+            acc[w] = Bf::mfma16(latent_operand<RL>(tile, part * kWindows + w, lane), pb, acc[w]);
+        buf ^= 1;
+    }
+    l += __shfl_xor(l, 16);
+    l += __shfl_xor(l, 32);
+    if (h0 + lo >= heads) return;
+    const int64_t row = (int64_t)b * heads + head;
+    float* dst = splits > 1 ? partial + (row * splits + sp) * (rank + 4) : nullptr;
+    if (dst && part == 0 && hi == 0) {
+        dst[rank] = m;
+        dst[rank + 1] = l;
+    }
+    const float inv = splits > 1 ? 1.f : 1.f / l;
+#pragma unroll
+    for (int w = 0; w < kWindows; ++w) {
+        const int d = 16 * (part * kWindows + w) + 4 * hi;
+        const float v[4] = {acc[w][0] * inv, acc[w][1] * inv, acc[w][2] * inv, acc[w][3] * inv};
+        if (rank % 4 == 0) {
+            if (d >= rank) continue;
+            if (dst) store_vec<Fp, 4>(dst + d, v);
+            else store_vec<Bf, 4>(out + row * rank + d, v);
+        } else {
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                if (d + r >= rank) continue;
+                if (dst) dst[d + r] = v[r];
+                else Bf::store(out + row * rank + d + r, v[r]);
+            }
+        }
+    }
+}
+
+// One workgroup per head; `splits` is at most 64, U of them are loaded together.
+template <int U>
+__global__ __launch_bounds__(512) void attn_merge_kernel(const float* __restrict__ partial, uint16_t* __restrict__ out,
                                                          int vdim, int splits) {
-    __shared__ float s_f[64];
+    __shared__ float s_share[64];
     const int64_t head = blockIdx.x;
     const float* p = partial + head * splits * (vdim + 4);
     if (threadIdx.x < 64) {
-        const int s = min((int)threadIdx.x, splits - 1);
-        const bool live = (int)threadIdx.x < splits;
+        const int s = min((int)threadIdx.x, splits - 1);           // lanes past the splits repeat the last
         const float m = p[s * (vdim + 4) + vdim], l = p[s * (vdim + 4) + vdim + 1];
-        const float mm = wave_max(m), f = live ? exp2_raw(m - mm) : 0.f;   // lanes past the splits repeat the last
-        s_f[threadIdx.x] = f / wave_sum(l * f);
+        const float mm = wave_max(m), f = (int)threadIdx.x < splits ? exp2_raw(m - mm) : 0.f;
+        s_share[threadIdx.x] = f / wave_sum(l * f);
     }
     __syncthreads();
-    for (int d = threadIdx.x; d < vdim; d += 256) {
+    for (int d = threadIdx.x; d < vdim; d += blockDim.x) {
         float at = 0.f;
-        for (int s0 = 0; s0 < splits; s0 += 8) {                   // eight loads in flight
-            float v[8];
+        for (int s0 = 0; s0 < splits; s0 += U) {
+            float v[U];
 #pragma unroll
-            for (int u = 0; u < 8; ++u) v[u] = p[min(s0 + u, splits - 1) * (vdim + 4) + d];
+            for (int u = 0; u < U; ++u) v[u] = p[min(s0 + u, splits - 1) * (vdim + 4) + d];
 #pragma unroll
-            for (int u = 0; u < 8; ++u) at += v[u] * (s0 + u < splits ? s_f[s0 + u] : 0.f);
+            for (int u = 0; u < U; ++u) at += v[u] * s_share[min(s0 + u, 63)];    // zero past the splits
         }
         Bf::store(out + head * vdim + d, at);
     }
+}
+
+void launch_merge(const void* partial, void* out, int64_t head_rows, int64_t vdim, int splits, void* stream) {
+    const auto kernel = splits <= 4 ? attn_merge_kernel<4> : splits <= 8 ? attn_merge_kernel<8> : attn_merge_kernel<16>;
+    kernel<<<dim3((unsigned)head_rows), dim3(vdim > 256 ? 512 : 256), 0, (hipStream_t)stream>>>(
+        (const float*)partial, (uint16_t*)out, (int)vdim, splits);
 }
 
 // Whether the matrix-core forms take this problem: bf16, equal cache rows of a width they exist for.
@@ -646,7 +769,6 @@ bool matrix_form(int64_t k_row, int64_t v_row, int dtype) {
     return dtype == NQH_BF16 && k_row == v_row &&
            (k_row == 32 || k_row == 64 || k_row == 96 || k_row == 128 || k_row == 192 || k_row == 256);
 }
-constexpr int kLatentWaves = 4;
 constexpr int decode_waves(int row) { return row > 128 ? 2 : 4; }
 int64_t most_keys(int64_t max_context, int64_t chunk, int64_t window) {
     const int64_t n = chunk > 0 ? std::min(chunk, max_context) : max_context;
@@ -762,14 +884,12 @@ extern "C" int nqh_attention_decode(const void* q, const void* k_cache, const vo
         if (groups > kMaxI32 || batch * heads > kMaxI32) return fail(NQH_ERR_ARG, fn, "problem too large");
         NQH_WITH_ROW(k_row, {
             constexpr int WAVES = decode_waves(R);
-            attn_decode_kernel<R, WAVES, 0><<<dim3((unsigned)groups), dim3(64 * WAVES), 0, (hipStream_t)stream>>>(
+            attn_decode_kernel<R, WAVES><<<dim3((unsigned)groups), dim3(64 * WAVES), 0, (hipStream_t)stream>>>(
                 (const uint16_t*)q, (const uint16_t*)k_cache, (const uint16_t*)v_cache, block_table, context_lens,
                 (const uint16_t*)sink, (uint16_t*)out, (float*)workspace, (int)heads, (int)kv_heads, (int)vdim, (int)block_size,
                 (int)max_blocks, (int)num_blocks, (int)chunk, (int)window, scale, splits, (int)head_tiles);
         });
-        if (splits > 1)
-            attn_merge_kernel<<<dim3((unsigned)(batch * heads)), dim3(256), 0, (hipStream_t)stream>>>(
-                (const float*)workspace, (uint16_t*)out, (int)vdim, splits);
+        if (splits > 1) launch_merge(workspace, out, batch * heads, vdim, splits, stream);
         return launched(fn);
     }
     NQH_WITH_TYPE(dtype, {
@@ -795,10 +915,11 @@ extern "C" int nqh_attention_decode(const void* q, const void* k_cache, const vo
         else if ((rr) == 32) { constexpr int RL = 512, R = 544; __VA_ARGS__; }                  \
         else { constexpr int RL = 512, R = 576; __VA_ARGS__; }                                  \
     } while (0)
-// Context splits: one workgroup per CU (that is what its LDS allows at the wide rows), at least a tile per wave.
+// Heads per workgroup are 16 or 32.  Context splits: two workgroups per CU, at least two tiles of 32 keys each.
+static int64_t latent_head_groups(int64_t heads) { return heads <= 16 ? 1 : cdiv(heads, 32); }
 static int latent_splits(int64_t batch, int64_t heads, int64_t longest) {
-    const int64_t want = 256 / std::max<int64_t>(1, batch * cdiv(heads, 16));
-    return (int)std::max<int64_t>(1, std::min({want, longest / (32 * kLatentWaves), (int64_t)64}));
+    const int64_t want = 512 / std::max<int64_t>(1, batch * latent_head_groups(heads));
+    return (int)std::max<int64_t>(1, std::min({want, longest / 64, (int64_t)64}));
 }
 static bool latent_matrix_form(int64_t rot_at, int64_t row, int dtype) {
     return dtype == NQH_BF16 && (rot_at == 64 || rot_at == 128 || rot_at == 256 || rot_at == 512) &&
@@ -835,22 +956,20 @@ extern "C" int nqh_latent_attention_decode(const void* q, const void* cache, con
         return launched(fn);
     }
     if (!aligned(q, 16) || !aligned(cache, 16)) return fail(NQH_ERR_ARG, fn, "misaligned pointer");
-    const int64_t head_tiles = cdiv(heads, 16);
+    const int64_t head_groups = latent_head_groups(heads);
     const int splits = latent_splits(batch, heads, block_size * max_blocks);
     const size_t need = splits > 1 ? (size_t)(batch * heads * splits * (rank + 4)) * sizeof(float) : 0;
     if (need && (!workspace || workspace_bytes < need || !aligned(workspace, 16)))
         return fail(NQH_ERR_WORKSPACE, fn, "workspace of %zu bytes needed, %zu given", need, workspace ? workspace_bytes : 0);
-    const int64_t groups = batch * head_tiles * splits;
+    const int64_t groups = batch * head_groups * splits;
     if (groups > kMaxI32 || batch * heads > kMaxI32) return fail(NQH_ERR_ARG, fn, "problem too large");
     NQH_WITH_LATENT(rot_at, row - rot_at, {
-        attn_decode_kernel<R, kLatentWaves, RL><<<dim3((unsigned)groups), dim3(64 * kLatentWaves), 0, (hipStream_t)stream>>>(
-            (const uint16_t*)q, (const uint16_t*)cache, (const uint16_t*)cache, block_table, context_lens,
-            (const uint16_t*)nullptr, (uint16_t*)out, (float*)workspace, (int)heads, 1, (int)rank, (int)block_size,
-            (int)max_blocks, (int)num_blocks, 0, 0, scale, splits, (int)head_tiles);
+        const auto kernel = heads <= 16 ? latent_decode_kernel<RL, R, 1> : latent_decode_kernel<RL, R, 2>;
+        kernel<<<dim3((unsigned)groups), dim3(256), 0, (hipStream_t)stream>>>(
+            (const uint16_t*)q, (const uint16_t*)cache, block_table, context_lens, (uint16_t*)out, (float*)workspace, (int)heads,
+            (int)rank, (int)block_size, (int)max_blocks, (int)num_blocks, scale, splits, (int)head_groups);
     });
-    if (splits > 1)
-        attn_merge_kernel<<<dim3((unsigned)(batch * heads)), dim3(256), 0, (hipStream_t)stream>>>(
-            (const float*)workspace, (uint16_t*)out, (int)rank, splits);
+    if (splits > 1) launch_merge(workspace, out, batch * heads, rank, splits, stream);
     return launched(fn);
 }
 

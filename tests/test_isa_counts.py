@@ -144,8 +144,6 @@ def test_hybrid_kernels_wait_for_their_tile_loads(tmp_path):
     asm = listing("attention")
     found = 0
     for name, ins in bodies(asm, "attn_decode_kernel"):
-        if not re.search(r"attn_decode_kernelILi\d+ELi\d+ELi0E", name):
-            continue                     # latent rows are key and value at once: one tile, waited for altogether
         loads = int(re.search(r"attn_decode_kernelILi(\d+)E", name).group(1)) // 16
         dma = [k for k, l in enumerate(ins) if "global_load_lds_dwordx4" in l]
         assert len(dma) == 2 * loads, (name, len(dma))
@@ -157,11 +155,11 @@ def test_hybrid_kernels_wait_for_their_tile_loads(tmp_path):
         found += 1
     assert found == 6
     found = 0
-    for source, kernel in (("attention", "attn_tile_kernel"), ("moe", "moe_gemm_kernel"), ("dense", "wide_linear_kernel")):
+    for source, kernel in (("attention", "attn_tile_kernel"), ("attention", "latent_decode_kernel"), ("moe", "moe_gemm_kernel"), ("dense", "wide_linear_kernel")):
         for name, ins in bodies(asm if source == "attention" else listing(source), kernel):
             first = next(k for k, l in enumerate(ins) if "v_mfma" in l)
             bar = max(k for k in range(first) if ins[k].startswith("s_barrier"))
             assert any("vmcnt(0)" in l for l in ins[bar - 4:bar]), name          # this stage's loads have landed
             assert not any("vmcnt(0)" in l for l in ins[bar:first]), name
             found += 1
-    assert found == 6 + 7 + 4 + 8       # attention over cache rows and over expanded latents, products
+    assert found == 6 + 7 + 16 + 4 + 8       # attention over cache rows, over expanded latents, over latents; products
