@@ -1,5 +1,6 @@
 // Dense linear for few rows: y = act(x W^T (+ bias)), bf16 operands, fp32 accumulation.
-//   up to 16 rows    skinny_linear_kernel: both operands straight from memory, the waves split the contraction
+//   up to 16 rows    skinny_linear_kernel: both operands straight from memory, the waves split the contraction; also for more
+//                    rows of few features, 16 at a time, where the next would leave most of the chip idle
 //   17 to 64 rows    wide_linear_kernel: the activations, by now as many bytes per workgroup as its weights, go through LDS
 #include "skinny.hpp"
 
@@ -12,7 +13,9 @@ __global__ __launch_bounds__(1024) void skinny_linear_kernel(const uint16_t* __r
                                                              int rows, int n_out, int n_in, int act, float param) {
     extern __shared__ __attribute__((aligned(16))) float s_sum[];
     const int lane = threadIdx.x & 63, lo = lane & 15, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-    const int waves = blockDim.x >> 6, n0 = blockIdx.x * 16;
+    const int waves = blockDim.x >> 6, n0 = blockIdx.x * 16, r0 = blockIdx.y * 16;
+    rows -= r0;
+    x += (int64_t)r0 * n_in;
     const uint16_t* w_row[1] = {w + (int64_t)min(n0 + lo, n_out - 1) * n_in};
     const uint16_t* x_row[1] = {x + (int64_t)min(lo, rows - 1) * n_in};
     f32x4 acc[1][1] = {{f32x4{0.f, 0.f, 0.f, 0.f}}};
@@ -21,8 +24,8 @@ __global__ __launch_bounds__(1024) void skinny_linear_kernel(const uint16_t* __r
     const int t = threadIdx.x >> 4, n = n0 + (threadIdx.x & 15);
     if (threadIdx.x < 256 && t < rows && n < n_out) {
         const float v = activation_f32(s_sum[threadIdx.x] + (bias ? Bf::to_f32(bias[n]) : 0.f), act, param);
-        if constexpr (F32OUT) reinterpret_cast<float*>(y)[(int64_t)t * n_out + n] = v;
-        else reinterpret_cast<uint16_t*>(y)[(int64_t)t * n_out + n] = Bf::from_f32(v);
+        if constexpr (F32OUT) reinterpret_cast<float*>(y)[(int64_t)(r0 + t) * n_out + n] = v;
+        else reinterpret_cast<uint16_t*>(y)[(int64_t)(r0 + t) * n_out + n] = Bf::from_f32(v);
     }
 }
 
@@ -130,7 +133,7 @@ extern "C" int nqh_skinny_linear(const void* x, const void* weight, const void* 
     if (act < NQH_ACT_NONE || act > NQH_ACT_SOFTCAP || (act == NQH_ACT_SOFTCAP && !(param > 0.f)))
         return fail(NQH_ERR_ARG, fn, "unknown activation, or a cap that is not positive");
     (void)hipGetLastError();
-    if (rows > 16) {
+    if (rows > 16 && out_features > 1024) {
         const bool narrow = out_features <= 8192;      // fewer features per workgroup: more workgroups
         if (rows <= 32)
             return narrow ? launch_wide<2, 2>(fn, x, weight, bias, y, rows, out_features, in_features, out_f32, act, param, stream)
@@ -139,9 +142,9 @@ extern "C" int nqh_skinny_linear(const void* x, const void* weight, const void* 
                       : launch_wide<4, 4>(fn, x, weight, bias, y, rows, out_features, in_features, out_f32, act, param, stream);
     }
     const int64_t groups = cdiv(out_features, 16);
-    const int waves = skinny_waves(groups, in_features);
+    const int waves = skinny_waves(groups * cdiv(rows, 16), in_features);
     const size_t lds = (size_t)waves * 256 * sizeof(float);
-    const dim3 grid((unsigned)groups), block((unsigned)waves * 64);
+    const dim3 grid((unsigned)groups, (unsigned)cdiv(rows, 16)), block((unsigned)waves * 64);
     if (out_f32)
         skinny_linear_kernel<true><<<grid, block, lds, (hipStream_t)stream>>>(
             (const uint16_t*)x, (const uint16_t*)weight, (const uint16_t*)bias, y, (int)rows, (int)out_features, (int)in_features, act,

@@ -74,7 +74,21 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(const typename T::elem* 
 }
 
 // Up to four taps: the weights and the rows that kConvRows tokens need are in registers before the first is used.
-constexpr int kConvRows = 8;
+constexpr int kConvRows = 16;
+// 16 bytes of a row as they lie in memory.
+template <typename T>
+struct Raw16;
+template <>
+struct Raw16<Bf> {
+    using type = u32x4;
+    static __device__ __forceinline__ float get(type v, int e) { return Bf::to_f32((uint16_t)(v[e >> 1] >> (16 * (e & 1)))); }
+};
+template <>
+struct Raw16<Fp> {
+    using type = f32x4;
+    static __device__ __forceinline__ float get(type v, int e) { return v[e]; }
+};
+
 template <typename T, int V>
 __global__ __launch_bounds__(256) void conv4_silu_kernel(const typename T::elem* __restrict__ x, int64_t x_stride,
                                                          const typename T::elem* __restrict__ w,
@@ -84,11 +98,13 @@ __global__ __launch_bounds__(256) void conv4_silu_kernel(const typename T::elem*
     const Piece pc = load_piece_desc(pieces, blockIdx.y);
     const int c = (blockIdx.x * 256 + threadIdx.x) * V, r0 = blockIdx.z * kConvRows;
     if (c >= channels || r0 >= pc.rows) return;
-    float v[kConvRows + 3][V], wt[4][V], b[V];
+    using Raw = Raw16<T>;
+    typename Raw::type v[kConvRows + 3];
+    float ahead[3][V], wt[4][V], b[V];
 #pragma unroll
     for (int j = 0; j < kConvRows + 3; ++j) {      // rows ahead of the sequence's tokens are replaced below
         const int at = min(r0 + j - 3, pc.rows - 1);
-        load_vec<T, V>(x + (int64_t)max(pc.first + at, pc.index == 0 ? pc.first : 0) * x_stride + c, v[j]);
+        v[j] = *reinterpret_cast<const typename Raw::type*>(x + (int64_t)max(pc.first + at, pc.index == 0 ? pc.first : 0) * x_stride + c);
     }
     load_vec<T, V>(bias + c, b);
 #pragma unroll
@@ -98,27 +114,32 @@ __global__ __launch_bounds__(256) void conv4_silu_kernel(const typename T::elem*
             const float f = T::load(w + (int64_t)(c + e) * taps + max(k - (4 - taps), 0));
             wt[k][e] = k >= 4 - taps ? f : 0.f;
         }
+#pragma unroll
+    for (int j = 0; j < 3; ++j)
+#pragma unroll
+        for (int e = 0; e < V; ++e) ahead[j][e] = Raw::get(v[j], e);
     if (r0 == 0 && pc.index == 0) {
 #pragma unroll
         for (int j = 0; j < 3; ++j) {
             const int k = j - (4 - taps);          // place in the stored inputs
 #pragma unroll
             for (int e = 0; e < V; ++e)
-                v[j][e] = k < 0 || pc.fresh ? 0.f : tail[((int64_t)pc.slot * (taps - 1) + k) * channels + c + e];
+                ahead[j][e] = k < 0 || pc.fresh ? 0.f : tail[((int64_t)pc.slot * (taps - 1) + k) * channels + c + e];
         }
     }
 #pragma unroll
     for (int j = 0; j < kConvRows; ++j) {
-        if (r0 + j >= pc.rows) return;
         float a[V];
 #pragma unroll
         for (int e = 0; e < V; ++e) {
-            a[e] = b[e];
-#pragma unroll
-            for (int k = 0; k < 4; ++k) a[e] += wt[k][e] * v[j + k][e];
+            const float now = Raw::get(v[j + 3], e);
+            a[e] = b[e] + wt[0][e] * ahead[0][e] + wt[1][e] * ahead[1][e] + wt[2][e] * ahead[2][e] + wt[3][e] * now;
+            ahead[0][e] = ahead[1][e];
+            ahead[1][e] = ahead[2][e];
+            ahead[2][e] = now;
             a[e] = silu_quick(a[e]);
         }
-        store_vec<T, V>(out + (int64_t)(pc.first + r0 + j) * channels + c, a);
+        if (r0 + j < pc.rows) store_vec<T, V>(out + (int64_t)(pc.first + r0 + j) * channels + c, a);
     }
 }
 
@@ -472,48 +493,65 @@ __global__ __launch_bounds__(256) void scan_chain_kernel(const float* __restrict
 }
 
 // ---- one token per sequence ------------------------------------------------------------------------------------------------
-// Workgroup: 64 channels of one row; its four waves share the states.
-template <typename T>
+// Workgroup: 64 channels of ROWS rows; its four waves share the states.
+template <typename T, int ROWS>
 __global__ __launch_bounds__(256) void scan_step_kernel(
     const typename T::elem* __restrict__ x, const float* __restrict__ dt, const typename T::elem* __restrict__ bc,
     int64_t bc_stride, const typename T::elem* __restrict__ z, int64_t z_stride, const typename T::elem* __restrict__ a_log,
     const typename T::elem* __restrict__ d_skip, float* __restrict__ state, const int32_t* __restrict__ slots,
-    const int64_t* __restrict__ positions, const uint8_t* __restrict__ active, typename T::elem* __restrict__ out, int num_slots,
-    int channels, int states) {
-    __shared__ float s_y[4][64];
-    const int row = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int64_t* __restrict__ positions, const uint8_t* __restrict__ active, typename T::elem* __restrict__ out, int batch,
+    int num_slots, int channels, int states) {
+    __shared__ float s_y[4][ROWS][64];
+    const int row0 = blockIdx.y * ROWS, lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int cw = blockIdx.x * 64 + lane, c = min(cw, channels - 1);
-    const int slot = slots[row];
-    const bool ok = active[row] && slot >= 0 && slot < num_slots, fresh = positions[row] <= 0;
-    const float d = dt[(int64_t)row * channels + c], xv = T::load(x + (int64_t)row * channels + c), dx = d * xv;
-    float y = 0.f;
-    if (ok) {
-        float* S = state + (int64_t)slot * states * channels + c;
-        const typename T::elem* B = bc + row * bc_stride;
-        for (int n0 = wave; n0 < states; n0 += 16) {              // four of this wave's states in flight
-            float s[4], a[4];
+    const int64_t size = (int64_t)states * channels;
+    int slot[ROWS];
+    bool ok[ROWS], fresh[ROWS];
+    float d[ROWS], dx[ROWS], y[ROWS];
 #pragma unroll
-            for (int u = 0; u < 4; ++u) {
-                const int n = min(n0 + 4 * u, states - 1);
-                s[u] = fresh ? 0.f : S[(int64_t)n * channels];
-                a[u] = T::load(a_log + (int64_t)c * states + n);
-            }
+    for (int r = 0; r < ROWS; ++r) {
+        const int row = min(row0 + r, batch - 1);
+        slot[r] = slots[row];
+        ok[r] = row0 + r < batch && active[row] && slot[r] >= 0 && slot[r] < num_slots;
+        fresh[r] = positions[row] <= 0;
+        slot[r] = ok[r] ? slot[r] : 0;
+        d[r] = dt[(int64_t)row * channels + c];
+        dx[r] = d[r] * T::load(x + (int64_t)row * channels + c);
+        y[r] = 0.f;
+    }
+    for (int n0 = wave; n0 < states; n0 += 16) {              // four of this wave's states of every row in flight
+        float s[ROWS][4], a[4];
 #pragma unroll
-            for (int u = 0; u < 4; ++u) {
-                const int n = n0 + 4 * u;
-                if (n < states) {
-                    const float v = __builtin_amdgcn_exp2f(d * (-expf(a[u]) * kLog2e)) * s[u] + dx * T::load(B + n);
-                    y += v * T::load(B + states + n);
-                    if (cw < channels) S[(int64_t)n * channels] = v;
-                }
+        for (int u = 0; u < 4; ++u) {
+            const int n = min(n0 + 4 * u, states - 1);
+            a[u] = T::load(a_log + (int64_t)c * states + n);
+#pragma unroll
+            for (int r = 0; r < ROWS; ++r) s[r][u] = state[slot[r] * size + (int64_t)n * channels + c];
+        }
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+            const int n = n0 + 4 * u;
+            if (n >= states) break;
+            const float A = -expf(a[u]) * kLog2e;
+#pragma unroll
+            for (int r = 0; r < ROWS; ++r) {
+                const typename T::elem* B = bc + min(row0 + r, batch - 1) * bc_stride;
+                const float v = __builtin_amdgcn_exp2f(d[r] * A) * (fresh[r] ? 0.f : s[r][u]) + dx[r] * T::load(B + n);
+                y[r] += v * T::load(B + states + n);
+                if (ok[r] && cw < channels) state[slot[r] * size + (int64_t)n * channels + c] = v;
             }
         }
     }
-    s_y[wave][lane] = y;
+#pragma unroll
+    for (int r = 0; r < ROWS; ++r) s_y[wave][r][lane] = y[r];
     __syncthreads();
-    if (wave == 0 && cw < channels) {
-        y = s_y[0][lane] + s_y[1][lane] + s_y[2][lane] + s_y[3][lane] + T::load(d_skip + c) * xv;
-        T::store(out + (int64_t)row * channels + c, ok ? y * silu_quick(T::load(z + row * z_stride + c)) : 0.f);
+    for (int r = wave; r < ROWS; r += 4) {
+        const int64_t row = row0 + r;
+        if (row >= batch || cw >= channels) continue;
+        const bool live = active[row] && slots[row] >= 0 && slots[row] < num_slots;
+        const float v = s_y[0][r][lane] + s_y[1][r][lane] + s_y[2][r][lane] + s_y[3][r][lane] +
+                        T::load(d_skip + c) * T::load(x + row * channels + c);
+        T::store(out + row * channels + c, live ? v * silu_quick(T::load(z + row * z_stride + c)) : 0.f);
     }
 }
 
@@ -557,17 +595,17 @@ extern "C" int nqh_conv_silu(const void* x, int64_t x_stride, const void* weight
     if (num_pieces <= 0 || num_pieces > 65535 || longest <= 0 || cdiv(longest, 8) > 65535 || x_stride < channels)
         return fail(NQH_ERR_ARG, fn, "1 to 65535 pieces, and x rows at least as wide as the channels");
     (void)hipGetLastError();
-#define NQH_GO(KERNEL, V)                                                                                                 \
-    KERNEL<T, V><<<dim3((unsigned)cdiv(channels, 256 * V), (unsigned)num_pieces, (unsigned)cdiv(longest, 8)), dim3(256), 0, \
+#define NQH_GO(KERNEL, V, ROWS)                                                                                            \
+    KERNEL<T, V><<<dim3((unsigned)cdiv(channels, 256 * V), (unsigned)num_pieces, (unsigned)cdiv(longest, ROWS)), dim3(256), 0, \
                    (hipStream_t)stream>>>((const E*)x, x_stride, (const E*)weight, (const E*)bias, tail, pieces, (E*)out,   \
                                           (int)channels, (int)taps)
     NQH_WITH_TYPE(dtype, {
         using E = typename T::elem;
         constexpr int V = 16 / sizeof(E);
         const bool vec = channels % V == 0 && x_stride % V == 0 && aligned(x, 16) && aligned(bias, 16) && aligned(out, 16);
-        if (taps <= 4 && vec) NQH_GO(conv4_silu_kernel, V);
-        else if (vec) NQH_GO(conv_silu_kernel, V);
-        else NQH_GO(conv_silu_kernel, 1);
+        if (taps <= 4 && vec) NQH_GO(conv4_silu_kernel, V, kConvRows);
+        else if (vec) NQH_GO(conv_silu_kernel, V, 8);
+        else NQH_GO(conv_silu_kernel, 1, 8);
     });
 #undef NQH_GO
     return launched(fn);
@@ -688,9 +726,11 @@ extern "C" int nqh_scan_step(const void* x, const float* dt, const void* bc, int
     (void)hipGetLastError();
     NQH_WITH_TYPE(dtype, {
         using E = typename T::elem;
-        scan_step_kernel<T><<<dim3((unsigned)cdiv(channels, 64), (unsigned)batch), dim3(256), 0, (hipStream_t)stream>>>(
+        const int rows = batch >= 32 ? 4 : 1;                 // several rows share the exponentials of a_log
+        const auto kernel = rows == 4 ? scan_step_kernel<T, 4> : scan_step_kernel<T, 1>;
+        kernel<<<dim3((unsigned)cdiv(channels, 64), (unsigned)cdiv(batch, rows)), dim3(256), 0, (hipStream_t)stream>>>(
             (const E*)x, dt, (const E*)bc, bc_stride, (const E*)z, z_stride, (const E*)a_log, (const E*)d_skip, state,
-            state_slots, positions, active, (E*)out, (int)num_slots, (int)channels, (int)states);
+            state_slots, positions, active, (E*)out, (int)batch, (int)num_slots, (int)channels, (int)states);
     });
     return launched(fn);
 }

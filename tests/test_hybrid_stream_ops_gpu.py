@@ -445,6 +445,28 @@ def test_one_state_entry_lives_on(dtype):
             assert (out[-1].float().cpu() - want).abs().max() < 2e-2 * want, (j, cuts)
 
 
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_scan_steps_of_a_wide_batch_equal_each_row_alone(dtype):
+    """More rows than one workgroup takes, some idle, fresh and running ones, slots in any order."""
+    B, C, N, rank, taps = 37, 100, 20, 8, 4
+    print(f"scan wide step {dtype}", flush=True)
+    xz, sel, conv, bias, up, dt_b, a_log, skip = (t.cuda() for t in scan_case(B, C, N, rank, taps, dtype))
+    s0, t0 = rand(B + 3, N, C, seed=5).cuda(), rand(B + 3, taps - 1, C, seed=6).cuda()
+    slot = torch.randperm(B + 3, generator=torch.Generator().manual_seed(3))[:B].to(torch.int32).cuda()
+    pos, active = torch.arange(B, device=DEV) % 5, torch.arange(B, device=DEV) % 7 != 3
+    dt = ops.scan_dt(sel[:, :rank], up, dt_b)
+
+    def go(rows, state, tail):
+        x = ops.conv_step(xz[rows, :C], conv, bias, tail, slot[rows], pos[rows], active[rows])
+        return ops.scan_step(x, dt[rows], sel[rows, rank:], xz[rows, C:], a_log, skip, state, slot[rows], pos[rows], active[rows])
+    sa, ta, sb, tb = s0.clone(), t0.clone(), s0.clone(), t0.clone()
+    got = go(slice(0, B), sa, ta)
+    want = torch.cat([go(slice(i, i + 1), sb, tb) for i in range(B)])
+    assert torch.equal(got, want) and torch.equal(sa, sb) and torch.equal(ta, tb)
+    idle = slot[~active].long()
+    assert torch.equal(sa[idle], s0[idle]) and torch.count_nonzero(got[~active]) == 0 and not torch.equal(sa, s0)
+
+
 def test_scan_ragged_pass_equals_each_sequence_alone():
     C, N, rank, taps, dtype = 80, 20, 8, 4, torch.bfloat16
     portions = [(0, 300), (37, 150), (0, 1), (250, 2), (128, 128), (5, 1)]
