@@ -14,8 +14,8 @@ the prefill GEMM TFLOP/s at the Qwen3-8B MLP shapes, the dequantise kernel, and 
 
 python bench.py [--gpus 1] [--steps K] [--warmup W] [--quick] [--no-cfg5] [--only-cfg5] [--no-cpu]
 
-python bench.py --hybrid [--hybrid-size SIZE]: instead of all that, prefill and decode throughput of hybrid decoders
-(Gafulix) beside AWQ Qwen3 models of the same layer sizes, random weights.
+python bench.py --hybrid [--hybrid-size SIZE] [--hybrid-model MODEL]: instead of all that, prefill and decode throughput of
+hybrid decoders (Gafulix, Roletar) beside AWQ Qwen3 models of the same layer sizes, random weights.
 
 For a profiler or a counter collection to look at one kernel (no timing, no JSON line):
 python bench.py --one linear|dequant|copy K N M [--one-dtype bf16|f16] [--one-iters 6] [--one-copies 1]
