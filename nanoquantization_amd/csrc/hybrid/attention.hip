@@ -664,7 +664,8 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(
 #pragma unroll
             for (int a = 0; a < 2; ++a) {
                 const int row = 16 * a + lo;
-                const unsigned char* p = s < RL / 32 ? tile + LL::at(row, 4 * s + hi) : tile + kRot + LR::at(row, 4 * (s - RL / 32) + hi);
+                const unsigned char* p = s < RL / 32 ? tile + LL::at(row, 4 * s + hi)
+                                                     : tile + kRot + LR::at(row, 4 * (s - RL / 32) + hi);
                 st[a] = Bf::mfma16(*reinterpret_cast<const u32x4*>(p), bq[s], st[a]);
             }
         float mx = kNegBig;

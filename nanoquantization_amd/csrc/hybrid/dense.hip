@@ -147,11 +147,11 @@ extern "C" int nqh_skinny_linear(const void* x, const void* weight, const void* 
     const dim3 grid((unsigned)groups, (unsigned)cdiv(rows, 16)), block((unsigned)waves * 64);
     if (out_f32)
         skinny_linear_kernel<true><<<grid, block, lds, (hipStream_t)stream>>>(
-            (const uint16_t*)x, (const uint16_t*)weight, (const uint16_t*)bias, y, (int)rows, (int)out_features, (int)in_features, act,
-            param);
+            (const uint16_t*)x, (const uint16_t*)weight, (const uint16_t*)bias, y, (int)rows, (int)out_features, (int)in_features,
+            act, param);
     else
         skinny_linear_kernel<false><<<grid, block, lds, (hipStream_t)stream>>>(
-            (const uint16_t*)x, (const uint16_t*)weight, (const uint16_t*)bias, y, (int)rows, (int)out_features, (int)in_features, act,
-            param);
+            (const uint16_t*)x, (const uint16_t*)weight, (const uint16_t*)bias, y, (int)rows, (int)out_features, (int)in_features,
+            act, param);
     return launched(fn);
 }

@@ -328,7 +328,7 @@ def head_linear(x: torch.Tensor, weight: torch.Tensor, y: torch.Tensor) -> torch
 
 
 def latent_prefill_query_row(dim: int, rot_dim: int, vdim: int, rank: int, dtype: torch.dtype) -> int:
-    """Width of a query row for latent_prefill_expanded; 0 if it does not take these sizes."""
+    """Width of a query row for latent_attention_prefill; 0 if it does not take these sizes."""
     if dtype not in _DTYPES or rank % 8:
         return 0
     return _lib.hybrid_lib().nqh_latent_attention_prefill_query_row(dim, rot_dim, vdim, _DTYPES[dtype])
